@@ -1,6 +1,7 @@
 /*
  * msgl_mix.h -- C ABI of the sequence-mixing kernels (latent attention, linear-recurrence layers, routed experts)
- * for gfx950; implemented by libmsgl_mix.so (mini-sglang_amd/csrc/seqmix.hip, mix_delta.hip, mix_par.hip).
+ * for gfx950; implemented by libmsgl_mix.so (mini-sglang_amd/csrc/seqmix.hip, mix_delta.hip, mix_par.hip,
+ * mix_scan.hip, mix_streams.hip).
  *
  * Same conventions as msgl_hip.h: raw device pointers, explicit sizes and strides in ELEMENTS, `stream` is a
  * hipStream_t passed as void*, every function returns 0 or a negative code and leaves a message for
@@ -27,7 +28,7 @@ extern "C" {
 #define MSGL_MIX_ACT_NONE 0
 #define MSGL_MIX_ACT_RELU2 1 /* max(z, 0)^2 */
 
-#define MSGL_MIX_ABI_VERSION 4
+#define MSGL_MIX_ABI_VERSION 5
 
 const char* msgl_mix_last_error(void);
 int msgl_mix_abi_version(void);
@@ -191,13 +192,14 @@ int msgl_mix_shift_norm(const float* x_in, float* x_out, const void* y0, int64_t
 int msgl_mix_commit_rows(float* dst, int64_t dst_stride, const float* src, int64_t src_stride, int layers, const int* slots, int batch, int W,
                          int* prev_tok, const int* ids, const int* cu_q, void* stream);
 
-/* Projection row [q: H x d | k: G x d | v: G x dv | ...] (+ bias: fp32, same layout, may be null): the first rot_dims entries of
- * every q and k head turn (cos_sin and pairing as in msgl_mix_latent_prep), with bit 0 of `unit` every q and k head, with bit 1
- * every v head is divided by its
- * root mean square; q -> q_out (fp32 [tokens, H * d]), k and v -> cache rows at out_loc ([slots, G * d], [slots, G * dv], T). */
+/* Projection row [q: H x d | k: G x d | v: Gv x dv | ...] (+ bias: fp32, same layout, may be null): with q_w / k_w (T [d], both or
+ * neither) every q / k head is RMS-normed and multiplied by that weight; then the first rot_dims entries of every q and k head turn
+ * (cos_sin and pairing as in msgl_mix_latent_prep); then, with bit 0 of `unit`, every q and k head and, with bit 1, every v head is
+ * divided by its root mean square; q -> q_out (fp32 [tokens, H * d]), k and v -> cache rows at out_loc ([slots, G * d], [slots,
+ * Gv * dv], T). */
 int msgl_mix_qk_prep(const void* proj, int64_t ld_proj, const float* bias, float* q_out, void* k_cache, void* v_cache, const int* out_loc,
-                     const int* positions, const float* cos_sin, int rot_dims, int interleaved, int unit, float eps, int tokens, int H,
-                     int G, int d, int dv, int dtype, void* stream);
+                     const int* positions, const float* cos_sin, int rot_dims, int interleaved, int unit, float eps, const void* q_w,
+                     const void* k_w, int tokens, int H, int G, int Gv, int d, int dv, int dtype, void* stream);
 
 /* Causal attention without normalisation over keys: out[t, h] = out_scale * sum_{j <= t} sigmoid(c(scale q_h . k_j) + pb[h]) v_j,
  * c(s) = softcap * tanh(s / softcap) (softcap <= 0: c(s) = s), query head h reads key/value head h / (H / G).  q: fp32 [tokens,
@@ -250,14 +252,24 @@ int msgl_mix_selective_scan(void* out, const void* x, int64_t ld_x, const void* 
                             const int* cu_q, const int* seq_lens, const int* slots, int batch, int C, int N, int dtype, int n_items,
                             const int* items, const int* item_first, float* scratch, void* stream);
 
-/* Softmax attention over the last `window` keys (window <= 0: all earlier keys) with a sink: out[t, h] = sum_j p_j v_j, p_j =
+/* Softmax attention over the last `window` keys (window <= 0: all earlier keys) and the first `keep` ones, with a sink: out[t, h] = sum_j p_j v_j, p_j =
  * exp(s_j) / (sum over visible keys of exp(s) + exp(sink[h])), s_j = scale q_h . k_j; sink fp32 [H] or null.  Query head h reads
  * key/value head h / (H / G).  q: fp32 [tokens, H * d]; caches and requests as in msgl_mix_sigmoid_attn; `splits` > 1 cuts the
  * visible keys into ranges joined by a second launch (workspace: fp32, msgl_mix_sink_attn_workspace_floats). */
 int msgl_mix_sink_attn_workspace_floats(int total_q, int H, int dv, int splits);
 int msgl_mix_sink_attn(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table,
                        int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G,
-                       int d, int dv, float scale, int window, const float* sink, int dtype, int splits, float* workspace, void* stream);
+                       int d, int dv, float scale, int window, int keep, const float* sink, int dtype, int splits, float* workspace,
+                       void* stream);
+
+/* The difference of two softmax maps over the same values: q [tokens, H, 2, d] (fp32), key rows [G, 2, d], value rows [G, dv]; with a1
+ * and a2 the outputs of the maps (same visible keys as above), o = a1 - lam[0] a2 (lam on the device), out[t, h] = o / sqrt(mean over
+ * dv of o^2 + eps) * post * sigmoid(gate[t, h]) (gate: T rows ld_gate apart, null: none).  Workspace for splits > 1:
+ * msgl_mix_sink_attn_workspace_floats of 2 H heads. */
+int msgl_mix_diff_attn(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table,
+                       int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G,
+                       int d, int dv, float scale, int window, int keep, const float* lam, float post, float eps, const void* gate,
+                       int64_t ld_gate, int dtype, int splits, float* workspace, void* stream);
 
 /* Router on fp32 logits z [tokens, E]: the `top` largest win (ties: lowest index), the weight of a choice is sigmoid(its logit)
  * -> ids int32 [tokens, top], wts fp32 [tokens, top]. */
@@ -276,6 +288,34 @@ int msgl_mix_sigmoid_gate(void* out, const float* o, const void* g, int64_t ld_g
 
 /* x <- cap * tanh(x / cap) in place (T rows of N, ld apart). */
 int msgl_mix_softcap(void* x, int64_t ld, int rows, int N, float cap, int dtype, void* stream);
+
+/* ---- multi-stream hybrid decoders (csrc/mix_streams.hip) ---- */
+
+/* Closes a sublayer and opens the next over `streams` (<= 16) residual streams, x: fp32 [rows, streams, W] (bcast: one row [rows, W]
+ * that stands for all).  With y (T [rows, W]): x'_t = sum_s mix[s * streams + t] x_s + out_w[t] y, else x' = x; x' -> x_out (fp32, may
+ * be x_in unless bcast; may be null).  u = sum_s read[s] x'_s (read null: ones);  h_out (T [rows, W], may be null) = (tanh(alpha[0] u)
+ * w + b) * scale, w and b T [W].  mix, out_w, read, alpha: fp32 on the device. */
+int msgl_mix_stream_norm(const float* x_in, int bcast, const void* y, const float* mix, const float* out_w, float* x_out, const float* read,
+                         const void* w, const void* b, const float* alpha, float scale, void* h_out, int rows, int streams, int W, int dtype,
+                         void* stream);
+
+/* Linear attention with decays per (request, head): S <- diag(a) S + k v^T, o = S^T q.  q, k [H x d], v, gate [H x dv]: T column blocks
+ * of rows `ld` apart; q and k are multiplied by q_scale / k_scale, after a rotation of their first rot_dims entries (cos_sin and
+ * pairing as in msgl_mix_latent_prep).  Either decay (fp32 [H]): a = decay[h]; or z (T [tokens, H x d], rows ld_z apart) and z_bias
+ * (fp32): log a = logsigmoid(z + z_bias) * inv_tau per key channel (no rotation then).  state: fp32 [slots, H, d, dv], row slots[b],
+ * zero for a request whose first new token is at position 0.  out: T rows of H x dv, every head RMS-normed (times w, T [dv], may be
+ * null) and multiplied by silu(gate); with `raw` fp32 o itself (the only form for heads
+ * msgl_mix_decay_attn_fused refuses).  n_items > 0: chunks as in
+ * msgl_mix_lightning; scratch: fp32, n_items * H * d * (dv + 1) floats.  d <= 256. */
+int msgl_mix_decay_attn_fused(int d, int dv);
+int msgl_mix_decay_attn(void* out, int64_t ld_out, int raw, const void* q, const void* k, const void* v, const void* gate, int64_t ld,
+                        const void* z, int64_t ld_z, const float* z_bias, float inv_tau, const float* decay, float q_scale, float k_scale,
+                        const float* cos_sin, const int* positions, int rot_dims, int interleaved, const void* w, float eps, float* state,
+                        const int* cu_q, const int* seq_lens, const int* slots, int batch, int H, int d, int dv, int dtype, int n_items,
+                        const int* items, const int* item_first, float* scratch, void* stream);
+
+/* gu: T rows [gate: N | up: N];  out (T [rows, N]) = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit). */
+int msgl_mix_clamp_gate(void* out, const void* gu, int rows, int N, float limit, float slope, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

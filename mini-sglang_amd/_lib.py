@@ -20,7 +20,7 @@ HIP_SO = LIB_DIR / "libmsgl_hip.so"
 COMM_SO = LIB_DIR / "libmsgl_comm.so"
 GEMM_SO = LIB_DIR / "libmsgl_gemm.so"
 MIX_SO = LIB_DIR / "libmsgl_mix.so"
-MIX_ABI_VERSION = 4
+MIX_ABI_VERSION = 5
 
 BF16, FP16, F32 = 0, 1, 2
 UNIQUE_ID_BYTES = 128
@@ -167,7 +167,7 @@ MIX_SIGNATURES = {
     "msgl_mix_embed_scaled": (_i, [_p, _p, _p, _p, _p, _p, _p, _i, _p, _f, _i, _i, _i, _i, _i, _i, _p]),
     "msgl_mix_shift_norm": (_i, [_p, _p, _p, _l, _p, _p, _l, _p, _p, _p, _f, _p, _p, _p, _p, _p, _p, _p, _p, _i, _f, _i, _i, _i, _p]),
     "msgl_mix_commit_rows": (_i, [_p, _l, _p, _l, _i, _p, _i, _i, _p, _p, _p, _p]),
-    "msgl_mix_qk_prep": (_i, [_p, _l, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f, _i, _i, _i, _i, _i, _i, _p]),
+    "msgl_mix_qk_prep": (_i, [_p, _l, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _f, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p]),
     "msgl_mix_sigmoid_attn_workspace_floats": (_i, [_i, _i, _i, _i]),
     "msgl_mix_sigmoid_attn": (_i, [_p, _l, _p, _p, _p, _p, _l, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _f, _p, _f, _i, _i, _p, _p]),
     "msgl_mix_ssd": (_i, [_p, _p, _l, _p, _l, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p]),
@@ -176,12 +176,18 @@ MIX_SIGNATURES = {
     "msgl_mix_norm_conv": (_i, [_p, _p, _p, _i, _p, _i, _f, _p, _p, _i, _f, _p, _i, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _p]),
     "msgl_mix_selective_scan": (_i, [_p, _p, _l, _p, _l, _p, _l, _p, _l, _p, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _p, _p, _p, _p]),
     "msgl_mix_sink_attn_workspace_floats": (_i, [_i, _i, _i, _i]),
-    "msgl_mix_sink_attn": (_i, [_p, _l, _p, _p, _p, _p, _l, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _p, _i, _i, _p, _p]),
+    "msgl_mix_sink_attn": (_i, [_p, _l, _p, _p, _p, _p, _l, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p, _i, _i, _p, _p]),
+    "msgl_mix_diff_attn": (_i, [_p, _l, _p, _p, _p, _p, _l, _p, _p, _p, _i, _i, _i, _i, _i, _i, _f, _i, _i, _p, _f, _f, _p, _l, _i, _i, _p, _p]),
     "msgl_mix_route_sigmoid": (_i, [_p, _p, _p, _i, _i, _i, _p]),
     "msgl_mix_scale_rows": (_i, [_p, _p, _p, _i, _i, _i, _i, _p]),
     "msgl_mix_route_scale": (_i, [_p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _p]),
     "msgl_mix_sigmoid_gate": (_i, [_p, _p, _p, _l, _i, _i, _i, _p]),
     "msgl_mix_softcap": (_i, [_p, _l, _i, _i, _f, _i, _p]),
+    "msgl_mix_stream_norm": (_i, [_p, _i, _p, _p, _p, _p, _p, _p, _p, _p, _f, _p, _i, _i, _i, _i, _p]),
+    "msgl_mix_decay_attn_fused": (_i, [_i, _i]),
+    "msgl_mix_decay_attn": (_i, [_p, _l, _i, _p, _p, _p, _p, _l, _p, _l, _p, _f, _p, _f, _f, _p, _p, _i, _i, _p, _f, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i,
+                                 _p, _p, _p, _p]),
+    "msgl_mix_clamp_gate": (_i, [_p, _p, _i, _i, _f, _f, _i, _p]),
 }
 
 

@@ -97,11 +97,11 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
 }
 
 template <typename T>
-const T* cp(const void* p) {
+__host__ __device__ const T* cp(const void* p) {
   return static_cast<const T*>(p);
 }
 template <typename T>
-T* mp(void* p) {
+__host__ __device__ T* mp(void* p) {
   return static_cast<T*>(p);
 }
 

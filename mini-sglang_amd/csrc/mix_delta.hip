@@ -797,7 +797,7 @@ __global__ __launch_bounds__(256) void head_gated_norm_kernel(T* __restrict__ ou
     const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
     for (int i = lane; i < dv; i += 64) {
       const float z = ld(g + (size_t)t * ld_g + h * dv + i);
-      st(out + ((size_t)t * H + h) * dv + i, oh[i] * inv * ld(w + i) * (act ? siluf_(z) : sigmoidf_(z)));
+      st(out + ((size_t)t * H + h) * dv + i, oh[i] * inv * (w ? ld(w + i) : 1.f) * (act ? siluf_(z) : sigmoidf_(z)));
     }
   }
 }
@@ -1018,7 +1018,7 @@ int msgl_mix_delta_rule(float* out, const float* qkv, float* state, const void* 
 
 int msgl_mix_head_gated_norm(void* out, const float* o, const void* gate, int64_t ld_gate, const void* w, float eps, int rows, int H,
                              int dv, int gate_act, int dtype, void* stream) {
-  MIX_REQUIRE(out && o && gate && w && rows >= 0 && H >= 1 && dv >= 1 && ld_gate >= (int64_t)H * dv && dtype_ok(dtype) &&
+  MIX_REQUIRE(out && o && gate && rows >= 0 && H >= 1 && dv >= 1 && ld_gate >= (int64_t)H * dv && dtype_ok(dtype) &&
                   (gate_act == 0 || gate_act == 1),
               "head_gated_norm: bad arguments");
   if (rows == 0) return MSGL_MIX_OK;

@@ -11,7 +11,8 @@
 //                           g = h + (h_prev - h) * shift with h_prev the previous token's h (same launch: recomputed from the
 //                           previous row; first token of a portion: the request's state row; position 0: zero)
 //   commit_rows_kernel      after the forward: every request's last h of every layer -> its state row; its last token id
-//   qk_prep_kernel          q, k (+ bias), rotation of the leading entries of each head, unit-RMS q and k; k, v -> cache rows
+//   qk_prep_kernel          q, k (+ bias), rotation of the leading entries of each head, unit-RMS q and k after it or a weighted RMS
+//                           norm before it; k, v -> cache rows
 //   sigmoid_attn_mfma_kernel  o[t, h] = sum_{j <= t} sigmoid(cap(scale q . k_j) + b_h) v_j, no normalisation over keys; bf16 caches,
 //                           both products on the matrix cores, weights in fp32; key ranges are plain partial sums
 //                           (sigmoid_merge_kernel adds them)
@@ -198,8 +199,8 @@ __global__ __launch_bounds__(256) void commit_rows_kernel(float* __restrict__ ds
 }
 
 // ------------------------------------------------------------------------------------------------ q / k preparation of grouped attention
-// One workgroup per token.  proj row = [q: H x d | k: G x d | v: G x dv | ...] (+ bias, fp32, same layout, may be null).  The first
-// rd entries of every q and k head turn by the token's angles (cos_sin row = cos | sin halves of rd / 2; pairs (2i, 2i + 1) when
+// One workgroup per token.  proj row = [q: H x d | k: G x d | v: Gv x dv | ...] (+ bias, fp32, same layout, may be null).  With q_w /
+// k_w (T [d] each, shared by the heads) every q / k head is first RMS-normed and multiplied by its weight.  The first rd entries of every q and k head then turn by the token's angles (cos_sin row = cos | sin halves of rd / 2; pairs (2i, 2i + 1) when
 // `interleaved`, else (i, i + rd / 2)); with bit 0 of `unit` every q and k head is then divided by its root mean square (eps inside
 // the root), with bit 1 every v head.
 // q -> q_out (fp32 [tokens, H * d]); k, v -> the cache rows at out_loc (T).
@@ -207,16 +208,33 @@ template <typename T>
 __global__ __launch_bounds__(256) void qk_prep_kernel(const T* __restrict__ proj, int64_t ld_proj, const float* __restrict__ bias,
                                                       float* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
                                                       const int* __restrict__ out_loc, const int* __restrict__ positions,
-                                                      const float* __restrict__ cos_sin, int rd, int interleaved, int unit, float eps, int H,
-                                                      int G, int d, int dv) {
-  extern __shared__ float row[];  // (H + G) * d
+                                                      const float* __restrict__ cos_sin, int rd, int interleaved, int unit, float eps,
+                                                      const T* __restrict__ q_w, const T* __restrict__ k_w, int H, int G, int Gv, int d,
+                                                      int dv) {
+  extern __shared__ float row[];  // (H + G) * d; with q_w / k_w another (H + G) * d of normed rows
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* src = proj + (size_t)t * ld_proj;
   const float* cs = cos_sin ? cos_sin + (size_t)positions[t] * rd : nullptr;
   const int half = rd >> 1, n = (H + G) * d;
+  const bool normed = q_w != nullptr;
+  float* pre = row + n;
+  if (normed) {
+    for (int hh = wave; hh < H + G; hh += 4) {
+      float ss = 0.f;
+      for (int i = lane; i < d; i += 64) {
+        const float v = ld(src + (size_t)hh * d + i) + (bias ? bias[(size_t)hh * d + i] : 0.f);
+        pre[hh * d + i] = v;
+        ss = fmaf(v, v, ss);
+      }
+      const float f = 1.0f / sqrtf(wave_sum(ss) / (float)d + eps);
+      const T* wt = hh < H ? q_w : k_w;
+      for (int i = lane; i < d; i += 64) pre[hh * d + i] *= f * ld(wt + i);
+    }
+    __syncthreads();
+  }
   for (int e = threadIdx.x; e < n; e += 256) {
     const int hh = e / d, j = e - hh * d;
-    auto in = [&](int jj) { return ld(src + (size_t)hh * d + jj) + (bias ? bias[(size_t)hh * d + jj] : 0.f); };
+    auto in = [&](int jj) { return normed ? pre[hh * d + jj] : ld(src + (size_t)hh * d + jj) + (bias ? bias[(size_t)hh * d + jj] : 0.f); };
     float v = in(j);
     if (j < rd) {
       if (interleaved) {
@@ -246,7 +264,7 @@ __global__ __launch_bounds__(256) void qk_prep_kernel(const T* __restrict__ proj
   for (int e = threadIdx.x; e < G * d; e += 256) st(k_cache + slot * G * d + e, row[H * d + e]);
   const size_t vo = (size_t)(H + G) * d;
   if (unit & 2) {  // every value head divided by its root mean square
-    for (int g = wave; g < G; g += 4) {
+    for (int g = wave; g < Gv; g += 4) {
       float ss = 0.f;
       for (int i = lane; i < dv; i += 64) {
         const float v = ld(src + vo + (size_t)g * dv + i) + (bias ? bias[vo + (size_t)g * dv + i] : 0.f);
@@ -254,11 +272,11 @@ __global__ __launch_bounds__(256) void qk_prep_kernel(const T* __restrict__ proj
       }
       const float f = 1.0f / sqrtf(wave_sum(ss) / (float)dv + eps);
       for (int i = lane; i < dv; i += 64)
-        st(v_cache + slot * G * dv + (size_t)g * dv + i, (ld(src + vo + (size_t)g * dv + i) + (bias ? bias[vo + (size_t)g * dv + i] : 0.f)) * f);
+        st(v_cache + slot * Gv * dv + (size_t)g * dv + i, (ld(src + vo + (size_t)g * dv + i) + (bias ? bias[vo + (size_t)g * dv + i] : 0.f)) * f);
     }
     return;
   }
-  for (int e = threadIdx.x; e < G * dv; e += 256) st(v_cache + slot * G * dv + e, ld(src + vo + e) + (bias ? bias[vo + e] : 0.f));
+  for (int e = threadIdx.x; e < Gv * dv; e += 256) st(v_cache + slot * Gv * dv + e, ld(src + vo + e) + (bias ? bias[vo + e] : 0.f));
 }
 
 // ------------------------------------------------------------------------------------------------ sigmoid attention
@@ -765,19 +783,21 @@ int msgl_mix_commit_rows(float* dst, int64_t dst_stride, const float* src, int64
 }
 
 int msgl_mix_qk_prep(const void* proj, int64_t ld_proj, const float* bias, float* q_out, void* k_cache, void* v_cache, const int* out_loc,
-                     const int* positions, const float* cos_sin, int rot_dims, int interleaved, int unit, float eps, int tokens, int H,
-                     int G, int d, int dv, int dtype, void* stream) {
+                     const int* positions, const float* cos_sin, int rot_dims, int interleaved, int unit, float eps, const void* q_w,
+                     const void* k_w, int tokens, int H, int G, int Gv, int d, int dv, int dtype, void* stream) {
   MIX_REQUIRE(proj && q_out && k_cache && v_cache && out_loc && dtype_ok(dtype), "qk_prep: null pointer / dtype");
-  MIX_REQUIRE(H >= 1 && G >= 1 && H % G == 0 && d >= 1 && dv >= 1 && rot_dims >= 0 && rot_dims <= d && rot_dims % 2 == 0,
+  MIX_REQUIRE(H >= 1 && G >= 1 && H % G == 0 && Gv >= 1 && d >= 1 && dv >= 1 && rot_dims >= 0 && rot_dims <= d && rot_dims % 2 == 0,
               "qk_prep: bad sizes H %d G %d d %d dv %d rot %d", H, G, d, dv, rot_dims);
   MIX_REQUIRE(rot_dims == 0 || (cos_sin && positions), "qk_prep: a rotation needs its table and positions");
-  MIX_REQUIRE(ld_proj >= (int64_t)(H + G) * d + (int64_t)G * dv, "qk_prep: projection row too short");
+  MIX_REQUIRE(ld_proj >= (int64_t)(H + G) * d + (int64_t)Gv * dv, "qk_prep: projection row too short");
+  MIX_REQUIRE((q_w == nullptr) == (k_w == nullptr), "qk_prep: norm weights for q and k, or for neither");
   if (tokens == 0) return MSGL_MIX_OK;
-  const size_t lds = (size_t)(H + G) * d * sizeof(float);
+  const size_t lds = (size_t)(H + G) * d * sizeof(float) * (q_w ? 2 : 1);
   hipStream_t s = static_cast<hipStream_t>(stream);
   DISPATCH_T(dtype, MIX_REQUIRE(ensure_lds((const void*)qk_prep_kernel<T>, lds) == 0, "qk_prep: heads do not fit LDS");
              hipLaunchKernelGGL(qk_prep_kernel<T>, dim3(tokens), dim3(256), lds, s, cp<T>(proj), ld_proj, bias, q_out, mp<T>(k_cache),
-                                mp<T>(v_cache), out_loc, positions, cos_sin, rot_dims, interleaved, unit, eps, H, G, d, dv);)
+                                mp<T>(v_cache), out_loc, positions, cos_sin, rot_dims, interleaved, unit, eps, cp<T>(q_w), cp<T>(k_w), H, G,
+                                Gv, d, dv);)
   MIX_LAUNCHED("qk_prep");
   return MSGL_MIX_OK;
 }

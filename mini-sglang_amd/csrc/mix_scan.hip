@@ -14,8 +14,10 @@
 //   selective_scan_kernel   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;  y_c = sum_n S[c, n] C_n + D_c x_c;  out = y silu(z);
 //                           a thread owns one channel's state row in registers; long portions as parallel chunks joined by
 //                           selective_join_kernel
-//   sink_attn_mfma_kernel   softmax attention over the last `window` keys with one more term exp(sink_h) in the denominator; bf16
-//                           caches, both products on the matrix cores, fp32 online softmax; key ranges + sink_merge_kernel
+//   sink_attn_mfma_kernel   softmax attention over the last `window` keys and the first `keep` ones, with one more term exp(sink_h) in
+//                           the denominator, or as the difference of two maps over the same values (normed and gated in the same
+//                           launch); bf16 caches, both products on the matrix cores, fp32 online softmax; key ranges +
+//                           sink_merge_kernel / diff_merge_kernel
 //   sink_attn_kernel        the same in plain fp32 (fp32 caches, heads past the matrix-core instances)
 //   route_sigmoid_kernel    the `top` largest router logits win, weights = sigmoid(logit)
 //   scale_rows_kernel       one copy of a token's row per chosen expert, multiplied by that choice's weight
@@ -419,27 +421,39 @@ __global__ __launch_bounds__(256) void selective_join_kernel(const float* __rest
 }
 
 // ------------------------------------------------------------------------------------------------ softmax attention with a window and a sink
-// Query head h reads key/value head h / (H / G); token i sees the keys j with 0 <= i - j < window (window <= 0: every j <= i);
+// Query head h reads key/value head h / (H / G); token i sees the keys j with 0 <= i - j < window (window <= 0: every j <= i) and the
+// first `keep` keys of the sequence (j < keep, j <= i);
 // weights = exp(score - max) / (sum over visible keys + exp(sink[h] - max)): the sink (may be null) has no key and no value.
+// MAPS = 2: a head has two query / key rows of d side by side (q [tokens, H, 2, d], key rows [G, 2, d]), each with a softmax of its own
+// over the same values; with their outputs a1 and a2, o = a1 - lam a2, o / sqrt(mean(o^2) + eps) * post * sigmoid(gate) leaves the kernel.
+// The visible keys of a workgroup are walked as one list: entry v is key v below `keep_eff` kept keys that lie before the window of the
+// workgroup's first token, and key v + (first windowed key - keep_eff) from there on.
 // A workgroup = 16 query rows (QT tokens of one request x HB query heads of ONE key/value head) x 16 lanes, one range of the
 // visible keys.  splits > 1: (max, sum, unnormalised output) per range, joined by sink_merge_kernel, where the sink enters.
 constexpr int kSinkRows = 16;
 constexpr int kSinkMaxC = 16;  // value columns per lane: dv <= 256
 
-template <typename T>
+struct DiffOut {  // what two maps become one output row with
+  const float* lam;  // one number on the device
+  const void* gate;  // T, rows ld_gate apart, columns as the output's; null: no gate
+  int64_t ld_gate;
+  float post, eps;
+};
+
+template <typename T, int MAPS>
 __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
                                                         float* __restrict__ part_ml, const float* __restrict__ q,
                                                         const T* __restrict__ k_cache, const T* __restrict__ v_cache,
                                                         const int* __restrict__ table, int64_t table_stride, const int* __restrict__ req_rows,
                                                         const int* __restrict__ seq_lens, const int* __restrict__ cu_q, int B, int total_q,
-                                                        int H, int G, int d, int dv, float scale, int window, const float* __restrict__ sink,
-                                                        int QT, int HB, int KT, int splits) {
+                                                        int H, int G, int d, int dv, float scale, int window, int keep,
+                                                        const float* __restrict__ sink, DiffOut df, int QT, int HB, int KT, int splits) {
   extern __shared__ float lds[];
-  const int qs = d + 1, vs = dv + 1;
-  float* sq = lds;                      // [16][d + 1]
-  float* sk = sq + kSinkRows * qs;      // [KT][d + 1]
+  const int dk = MAPS * d, qs = dk + 1, vs = dv + 1;
+  float* sq = lds;                      // [16][MAPS d + 1]
+  float* sk = sq + kSinkRows * qs;      // [KT][MAPS d + 1]
   float* sv = sk + KT * qs;             // [KT][dv + 1]
-  float* sp = sv + KT * vs;             // [16][KT]
+  float* sp = sv + KT * vs;             // [MAPS][16][KT]
   __shared__ int s_req, s_tok0, s_cnt[256];
   find_group(cu_q, B, QT, s_cnt, &s_req, &s_tok0);
   const int b = s_req;
@@ -458,88 +472,128 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
   const int last_tok = min(s_tok0 + QT, q_len) - 1;
   const int n_keys = start + last_tok + 1;
   const int lo_blk = window > 0 ? max(0, start + s_tok0 - window + 1) : 0;
-  const int per = ((n_keys - lo_blk + splits - 1) / splits + KT - 1) / KT * KT;
-  const int k_begin = lo_blk + blockIdx.z * per, k_end = min(n_keys, k_begin + per);
-  for (int i = l; i < d; i += 16) sq[r * qs + i] = q[((size_t)tok * H + head) * d + i];
+  const int keep_eff = min(keep, lo_blk), shift = lo_blk - keep_eff, n_vis = n_keys - shift;
+  const int per = ((n_vis + splits - 1) / splits + KT - 1) / KT * KT;
+  const int k_begin = blockIdx.z * per, k_end = min(n_vis, k_begin + per);
+  for (int i = l; i < dk; i += 16) sq[r * qs + i] = q[((size_t)tok * H + head) * dk + i];
   const int* trow = table + (size_t)req_rows[b] * table_stride;
-  float o[kSinkMaxC];
+  float o[MAPS][kSinkMaxC], m[MAPS], lsum[MAPS];
 #pragma unroll
-  for (int i = 0; i < kSinkMaxC; ++i) o[i] = 0.f;
-  float m = -INFINITY, lsum = 0.f;
-  const int nkd = G * d, nvd = G * dv;
+  for (int a = 0; a < MAPS; ++a) {
+#pragma unroll
+    for (int i = 0; i < kSinkMaxC; ++i) o[a][i] = 0.f;
+    m[a] = -INFINITY;
+    lsum[a] = 0.f;
+  }
+  const int nkd = G * dk, nvd = G * dv;
+  auto key_at = [&](int v) { return v < keep_eff ? v : v + shift; };
   for (int j0 = k_begin; j0 < k_end; j0 += KT) {
     __syncthreads();
     const int nk = min(KT, k_end - j0);
-    for (int e = threadIdx.x; e < nk * d; e += 256) {
-      const int j = e / d, i = e - j * d;
-      sk[j * qs + i] = ld(k_cache + (size_t)trow[j0 + j] * nkd + (size_t)kvh * d + i);
+    for (int e = threadIdx.x; e < nk * dk; e += 256) {
+      const int j = e / dk, i = e - j * dk;
+      sk[j * qs + i] = ld(k_cache + (size_t)trow[key_at(j0 + j)] * nkd + (size_t)kvh * dk + i);
     }
     for (int e = threadIdx.x; e < nk * dv; e += 256) {
       const int j = e / dv, i = e - j * dv;
-      sv[j * vs + i] = ld(v_cache + (size_t)trow[j0 + j] * nvd + (size_t)kvh * dv + i);
+      sv[j * vs + i] = ld(v_cache + (size_t)trow[key_at(j0 + j)] * nvd + (size_t)kvh * dv + i);
     }
     __syncthreads();
-    float tmax = -INFINITY;
-    for (int j = l; j < KT; j += 16) {
-      float s = -INFINITY;
-      if (j < nk && j0 + j <= limit && j0 + j >= lo_row) {
-        float acc = 0.f;
-        const float* qp = sq + r * qs;
-        const float* kp = sk + j * qs;
-        for (int i = 0; i < d; ++i) acc = fmaf(qp[i], kp[i], acc);
-        s = acc * scale;
+    float alpha[MAPS];
+#pragma unroll
+    for (int a = 0; a < MAPS; ++a) {
+      float* spa = sp + (size_t)a * kSinkRows * KT;
+      float tmax = -INFINITY;
+      for (int j = l; j < KT; j += 16) {
+        float s = -INFINITY;
+        const int key = key_at(j0 + j);
+        if (j < nk && key <= limit && (key >= lo_row || key < keep)) {
+          float acc = 0.f;
+          const float* qp = sq + r * qs + a * d;
+          const float* kp = sk + j * qs + a * d;
+          for (int i = 0; i < d; ++i) acc = fmaf(qp[i], kp[i], acc);
+          s = acc * scale;
+        }
+        spa[r * KT + j] = s;
+        tmax = fmaxf(tmax, s);
       }
-      sp[r * KT + j] = s;
-      tmax = fmaxf(tmax, s);
-    }
 #pragma unroll
-    for (int x = 8; x >= 1; x >>= 1) tmax = fmaxf(tmax, __shfl_xor(tmax, x, 64));
-    const float m_new = fmaxf(m, tmax);
-    const float alpha = m_new == -INFINITY ? 1.0f : expf(m - m_new);
-    float psum = 0.f;
-    for (int j = l; j < KT; j += 16) {
-      const float s = sp[r * KT + j];
-      const float p = s == -INFINITY ? 0.f : expf(s - m_new);
-      sp[r * KT + j] = p;
-      psum += p;
-    }
+      for (int x = 8; x >= 1; x >>= 1) tmax = fmaxf(tmax, __shfl_xor(tmax, x, 64));
+      const float m_new = fmaxf(m[a], tmax);
+      alpha[a] = m_new == -INFINITY ? 1.0f : expf(m[a] - m_new);
+      float psum = 0.f;
+      for (int j = l; j < KT; j += 16) {
+        const float s = spa[r * KT + j];
+        const float p = s == -INFINITY ? 0.f : expf(s - m_new);
+        spa[r * KT + j] = p;
+        psum += p;
+      }
 #pragma unroll
-    for (int x = 8; x >= 1; x >>= 1) psum += __shfl_xor(psum, x, 64);
-    lsum = fmaf(lsum, alpha, psum);
-    m = m_new;
+      for (int x = 8; x >= 1; x >>= 1) psum += __shfl_xor(psum, x, 64);
+      lsum[a] = fmaf(lsum[a], alpha[a], psum);
+      m[a] = m_new;
+    }
     __syncthreads();
+#pragma unroll
+    for (int a = 0; a < MAPS; ++a)
+#pragma unroll
+      for (int i = 0; i < kSinkMaxC; ++i) {
+        const int c = l + 16 * i;
+        if (c < dv) {
+          float acc = o[a][i] * alpha[a];
+          for (int j = 0; j < nk; ++j) acc = fmaf(sp[(a * kSinkRows + r) * KT + j], sv[j * vs + c], acc);
+          o[a][i] = acc;
+        }
+      }
+  }
+  if (MAPS == 2 && splits == 1) {
+    const float f0 = 1.0f / lsum[0], f1 = df.lam[0] / lsum[MAPS - 1];  // a row that is not valid holds no sum and is not written
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < kSinkMaxC; ++i) {
+      o[0][i] = o[0][i] * f0 - o[MAPS - 1][i] * f1;
+      if (l + 16 * i < dv) ss = fmaf(o[0][i], o[0][i], ss);
+    }
+#pragma unroll
+    for (int x = 8; x >= 1; x >>= 1) ss += __shfl_xor(ss, x, 64);
+    if (!valid) return;
+    const float f = df.post / sqrtf(ss / (float)dv + df.eps);
+    const T* gate = cp<T>(df.gate);
 #pragma unroll
     for (int i = 0; i < kSinkMaxC; ++i) {
       const int c = l + 16 * i;
       if (c < dv) {
-        float acc = o[i] * alpha;
-        for (int j = 0; j < nk; ++j) acc = fmaf(sp[r * KT + j], sv[j * vs + c], acc);
-        o[i] = acc;
+        const float gz = gate ? sigmoidf_(ld(gate + (size_t)tok * df.ld_gate + (size_t)head * dv + c)) : 1.f;
+        st(out + (size_t)tok * ld_out + (size_t)head * dv + c, o[0][i] * f * gz);
       }
     }
+    return;
   }
   if (!valid) return;
   if (splits == 1) {
     const float sk_h = sink ? sink[head] : -INFINITY;
-    const float mf = fmaxf(m, sk_h);
-    const float em = expf(m - mf);
-    const float f = em / (lsum * em + (sink ? expf(sk_h - mf) : 0.f));
+    const float mf = fmaxf(m[0], sk_h);
+    const float em = expf(m[0] - mf);
+    const float f = em / (lsum[0] * em + (sink ? expf(sk_h - mf) : 0.f));
 #pragma unroll
     for (int i = 0; i < kSinkMaxC; ++i) {
       const int c = l + 16 * i;
-      if (c < dv) st(out + (size_t)tok * ld_out + (size_t)head * dv + c, o[i] * f);
+      if (c < dv) st(out + (size_t)tok * ld_out + (size_t)head * dv + c, o[0][i] * f);
     }
     return;
   }
 #pragma unroll
-  for (int i = 0; i < kSinkMaxC; ++i) {
-    const int c = l + 16 * i;
-    if (c < dv) part_o[((size_t)blockIdx.z * total_q + tok) * H * dv + (size_t)head * dv + c] = o[i];
-  }
-  if (l == 0) {
-    float* ml = part_ml + (((size_t)blockIdx.z * total_q + tok) * H + head) * 2;
-    ml[0] = m;
-    ml[1] = lsum;
+  for (int a = 0; a < MAPS; ++a) {
+    const size_t row = (((size_t)blockIdx.z * total_q + tok) * H + head) * MAPS + a;
+#pragma unroll
+    for (int i = 0; i < kSinkMaxC; ++i) {
+      const int c = l + 16 * i;
+      if (c < dv) part_o[row * dv + c] = o[a][i];
+    }
+    if (l == 0) {
+      part_ml[row * 2] = m[a];
+      part_ml[row * 2 + 1] = lsum[a];
+    }
   }
 }
 
@@ -553,16 +607,16 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
 //   tile (ds_read_b64_tr_b16).
 constexpr int kNKT = 64;
 
-template <int KC, int VC>
+template <int KC, int VC, int MAPS>
 __global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
                                                              float* __restrict__ part_ml, const float* __restrict__ q,
                                                              const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
                                                              const int* __restrict__ table, int64_t table_stride,
                                                              const int* __restrict__ req_rows, const int* __restrict__ seq_lens,
                                                              const int* __restrict__ cu_q, int B, int total_q, int H, int G, int d, int dv,
-                                                             float scale, int window, const float* __restrict__ sink, int QT, int HB,
-                                                             int splits, int kvec, int vvec) {
-  constexpr int KS = KC * 32 + 8, VS = VC * 16 + 8;
+                                                             float scale, int window, int keep, const float* __restrict__ sink, DiffOut df, int QT,
+                                                             int HB, int splits, int kvec, int vvec) {
+  constexpr int KM = KC * 32, KS = MAPS * KM + 8, VS = VC * 16 + 8;
   extern __shared__ __attribute__((aligned(16))) uint16_t smem[];
   uint16_t* sk = smem;               // [kNKT][KS]
   uint16_t* sv = smem + kNKT * KS;   // [kNKT][VS]
@@ -587,35 +641,42 @@ __global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict_
   const int last_tok = min(s_tok0 + QT, q_len) - 1;
   const int n_keys = start + last_tok + 1;
   const int lo_blk = window > 0 ? max(0, start + s_tok0 - window + 1) : 0;
-  const int per = ((n_keys - lo_blk + splits - 1) / splits + kNKT - 1) / kNKT * kNKT;
-  const int k_begin = lo_blk + z * per, k_end = min(n_keys, k_begin + per);
+  const int keep_eff = min(keep, lo_blk), shift = lo_blk - keep_eff, n_vis = n_keys - shift;
+  const int per = ((n_vis + splits - 1) / splits + kNKT - 1) / kNKT * kNKT;
+  const int k_begin = z * per, k_end = min(n_vis, k_begin + per);
+  auto key_at = [&](int v) { return v < keep_eff ? v : v + shift; };
   const bool wave_live = __builtin_amdgcn_ballot_w64(valid) != 0;
-  bf16x8_t qf[KC];
-  {
-    const float* qrow = q + ((size_t)tok * H + head) * d;
+  bf16x8_t qf[MAPS][KC];
+  f32x4_t o[MAPS][VC];
+  float m[MAPS], lsum[MAPS];  // the row's maximum (the same in its four lanes) and this lane's share of the row's sum
+#pragma unroll
+  for (int a = 0; a < MAPS; ++a) {
+    const float* qrow = q + (((size_t)tok * H + head) * MAPS + a) * d;
 #pragma unroll
     for (int kc = 0; kc < KC; ++kc) {
       const int k = kc * 32 + lg * 8;
       Q4 v = (valid && k < d) ? load8(qrow + k, d - k, (d & 3) == 0) : Q4{0u, 0u, 0u, 0u};
-      qf[kc] = __builtin_bit_cast(bf16x8_t, v);
+      qf[a][kc] = __builtin_bit_cast(bf16x8_t, v);
     }
-  }
-  f32x4_t o[VC];
 #pragma unroll
-  for (int vt = 0; vt < VC; ++vt) o[vt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, lsum = 0.f;  // the row's maximum (the same in its four lanes) and this lane's share of the row's sum
+    for (int vt = 0; vt < VC; ++vt) o[a][vt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    m[a] = -INFINITY;
+    lsum[a] = 0.f;
+  }
   const int* trow = table + (size_t)req_rows[b] * table_stride;
-  const size_t nkd = (size_t)G * d, nvd = (size_t)G * dv, ko = (size_t)kvh * d, vo = (size_t)kvh * dv;
+  const size_t nkd = (size_t)G * MAPS * d, nvd = (size_t)G * dv, ko = (size_t)kvh * MAPS * d, vo = (size_t)kvh * dv;
   // the next tile's rows are requested before the current tile's products: their latency hides under the MFMAs
-  constexpr int NK = (kNKT * KC * 4 + 255) / 256, NV = (kNKT * VC * 2 + 255) / 256;
+  constexpr int KCH = MAPS * KC * 4;  // 16-byte pieces of a key row
+  constexpr int NK = (kNKT * KCH + 255) / 256, NV = (kNKT * VC * 2 + 255) / 256;
   Q4 pre_k[NK], pre_v[NV];
   auto request = [&](int j0, int buf) {
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int e = u * 256 + threadIdx.x;
-      const int key = e / (KC * 4), k = (e - key * (KC * 4)) * 8;
+      const int key = e / KCH, ch = e - key * KCH, a = ch / (KC * 4), k = (ch - a * (KC * 4)) * 8;
       pre_k[u] = Q4{0u, 0u, 0u, 0u};
-      if (e < kNKT * KC * 4 && j0 + key < k_end && k < d) pre_k[u] = load8(k_cache + (size_t)s_slot[buf][key] * nkd + ko + k, d - k, kvec != 0);
+      if (e < kNKT * KCH && j0 + key < k_end && k < d)
+        pre_k[u] = load8(k_cache + (size_t)s_slot[buf][key] * nkd + ko + (size_t)a * d + k, d - k, kvec != 0);
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
@@ -625,18 +686,18 @@ __global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict_
       if (e < kNKT * VC * 2 && j0 + key < k_end && c < dv) pre_v[u] = load8(v_cache + (size_t)s_slot[buf][key] * nvd + vo + c, dv - c, vvec != 0);
     }
   };
-  if (threadIdx.x < kNKT && k_begin + (int)threadIdx.x < k_end) s_slot[0][threadIdx.x] = trow[k_begin + threadIdx.x];
+  if (threadIdx.x < kNKT && k_begin + (int)threadIdx.x < k_end) s_slot[0][threadIdx.x] = trow[key_at(k_begin + threadIdx.x)];
   __syncthreads();
   if (k_begin < k_end) request(k_begin, 0);
   int buf = 0;
   for (int j0 = k_begin; j0 < k_end; j0 += kNKT, buf ^= 1) {
     __syncthreads();
-    if (threadIdx.x < kNKT && j0 + kNKT + (int)threadIdx.x < k_end) s_slot[buf ^ 1][threadIdx.x] = trow[j0 + kNKT + threadIdx.x];
+    if (threadIdx.x < kNKT && j0 + kNKT + (int)threadIdx.x < k_end) s_slot[buf ^ 1][threadIdx.x] = trow[key_at(j0 + kNKT + threadIdx.x)];
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int e = u * 256 + threadIdx.x;
-      const int key = e / (KC * 4), ch = e - key * (KC * 4);
-      if (e < kNKT * KC * 4) *reinterpret_cast<Q4*>(&sk[key * KS + ch * 8]) = pre_k[u];
+      const int key = e / KCH, ch = e - key * KCH;
+      if (e < kNKT * KCH) *reinterpret_cast<Q4*>(&sk[key * KS + ch * 8]) = pre_k[u];
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
@@ -648,48 +709,51 @@ __global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict_
     if (j0 + kNKT < k_end) request(j0 + kNKT, buf ^ 1);
     if (!wave_live) continue;
     constexpr int NKS = kNKT / 16;
-    f32x4_t sc[NKS];
-    float tmax = -INFINITY;
+    s16x4_t pf[MAPS][NKS];
 #pragma unroll
-    for (int ks = 0; ks < NKS; ++ks) {
-      f32x4_t sacc{0.f, 0.f, 0.f, 0.f};
+    for (int a = 0; a < MAPS; ++a) {
+      f32x4_t sc[NKS];
+      float tmax = -INFINITY;
 #pragma unroll
-      for (int kc = 0; kc < KC; ++kc) {
-        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&sk[(ks * 16 + lr) * KS + kc * 32 + lg * 8]);
-        sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[kc], sacc, 0, 0, 0);
+      for (int ks = 0; ks < NKS; ++ks) {
+        f32x4_t sacc{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kc = 0; kc < KC; ++kc) {
+          const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&sk[(ks * 16 + lr) * KS + a * KM + kc * 32 + lg * 8]);
+          sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[a][kc], sacc, 0, 0, 0);
+        }
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          const int v = j0 + ks * 16 + 4 * lg + c, j = key_at(v);
+          const float s = (j <= limit && (j >= lo_row || j < keep) && v < k_end) ? sacc[c] * scale : -INFINITY;
+          sacc[c] = s;
+          tmax = fmaxf(tmax, s);
+        }
+        sc[ks] = sacc;
       }
+      tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
+      tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
+      const float m_new = fmaxf(m[a], tmax);
+      const float alpha = m_new == -INFINITY ? 1.0f : __expf(m[a] - m_new);
+      float psum = 0.f;
 #pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        const int j = j0 + ks * 16 + 4 * lg + c;
-        const float s = (j <= limit && j >= lo_row && j < k_end) ? sacc[c] * scale : -INFINITY;
-        sacc[c] = s;
-        tmax = fmaxf(tmax, s);
+      for (int ks = 0; ks < NKS; ++ks) {
+        float pe[4];
+#pragma unroll
+        for (int c = 0; c < 4; ++c) {
+          pe[c] = sc[ks][c] == -INFINITY ? 0.f : __expf(sc[ks][c] - m_new);
+          psum += pe[c];
+        }
+        const uint32_t p01 = bf16_bits(pe[0]) | (bf16_bits(pe[1]) << 16), p23 = bf16_bits(pe[2]) | (bf16_bits(pe[3]) << 16);
+        pf[a][ks] = __builtin_bit_cast(s16x4_t, uint2{p01, p23});
       }
-      sc[ks] = sacc;
+      lsum[a] = fmaf(lsum[a], alpha, psum);
+      m[a] = m_new;
+#pragma unroll
+      for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) o[a][vt][c] *= alpha;
     }
-    tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
-    tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
-    const float m_new = fmaxf(m, tmax);
-    const float alpha = m_new == -INFINITY ? 1.0f : __expf(m - m_new);
-    s16x4_t pf[NKS];
-    float psum = 0.f;
-#pragma unroll
-    for (int ks = 0; ks < NKS; ++ks) {
-      float pe[4];
-#pragma unroll
-      for (int c = 0; c < 4; ++c) {
-        pe[c] = sc[ks][c] == -INFINITY ? 0.f : __expf(sc[ks][c] - m_new);
-        psum += pe[c];
-      }
-      const uint32_t p01 = bf16_bits(pe[0]) | (bf16_bits(pe[1]) << 16), p23 = bf16_bits(pe[2]) | (bf16_bits(pe[3]) << 16);
-      pf[ks] = __builtin_bit_cast(s16x4_t, uint2{p01, p23});
-    }
-    lsum = fmaf(lsum, alpha, psum);
-    m = m_new;
-#pragma unroll
-    for (int vt = 0; vt < VC; ++vt)
-#pragma unroll
-      for (int c = 0; c < 4; ++c) o[vt][c] *= alpha;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks) {
       if (j0 + ks * 16 >= k_end) break;
@@ -697,38 +761,72 @@ __global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict_
 #pragma unroll
       for (int vt = 0; vt < VC; ++vt) {
         const s16x4_t vf = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)(vbase + vt * 16));
-        o[vt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pf[ks], o[vt], 0, 0, 0);
+#pragma unroll
+        for (int a = 0; a < MAPS; ++a) o[a][vt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pf[a][ks], o[a][vt], 0, 0, 0);
       }
     }
   }
-  lsum += __shfl_xor(lsum, 16, 64);
-  lsum += __shfl_xor(lsum, 32, 64);
-  if (!valid) return;
-  if (splits == 1) {
-    const float sk_h = sink ? sink[head] : -INFINITY;
-    const float mf = fmaxf(m, sk_h);
-    const float em = __expf(m - mf);
-    const float f = em / (lsum * em + (sink ? __expf(sk_h - mf) : 0.f));
+#pragma unroll
+  for (int a = 0; a < MAPS; ++a) {
+    lsum[a] += __shfl_xor(lsum[a], 16, 64);
+    lsum[a] += __shfl_xor(lsum[a], 32, 64);
+  }
+  if (MAPS == 2 && splits == 1) {
+    const float f0 = 1.0f / lsum[0], f1 = df.lam[0] / lsum[MAPS - 1];  // a row that is not valid holds no sum and is not written
+    float ss = 0.f;
+#pragma unroll
+    for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        o[0][vt][c] = o[0][vt][c] * f0 - o[MAPS - 1][vt][c] * f1;
+        ss = fmaf(o[0][vt][c], o[0][vt][c], ss);  // columns past dv are zero
+      }
+    ss += __shfl_xor(ss, 16, 64);
+    ss += __shfl_xor(ss, 32, 64);
+    if (!valid) return;
+    const float f = df.post / sqrtf(ss / (float)dv + df.eps);
+    const bf16_t* gate = cp<bf16_t>(df.gate);
 #pragma unroll
     for (int vt = 0; vt < VC; ++vt)
 #pragma unroll
       for (int c = 0; c < 4; ++c) {
         const int v = vt * 16 + 4 * lg + c;
-        if (v < dv) st(out + (size_t)tok * ld_out + (size_t)head * dv + v, o[vt][c] * f);
+        if (v < dv) {
+          const float gz = gate ? 1.0f / (1.0f + __expf(-ld(gate + (size_t)tok * df.ld_gate + (size_t)head * dv + v))) : 1.f;
+          st(out + (size_t)tok * ld_out + (size_t)head * dv + v, o[0][vt][c] * f * gz);
+        }
+      }
+    return;
+  }
+  if (!valid) return;
+  if (splits == 1) {
+    const float sk_h = sink ? sink[head] : -INFINITY;
+    const float mf = fmaxf(m[0], sk_h);
+    const float em = __expf(m[0] - mf);
+    const float f = em / (lsum[0] * em + (sink ? __expf(sk_h - mf) : 0.f));
+#pragma unroll
+    for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        const int v = vt * 16 + 4 * lg + c;
+        if (v < dv) st(out + (size_t)tok * ld_out + (size_t)head * dv + v, o[0][vt][c] * f);
       }
     return;
   }
 #pragma unroll
-  for (int vt = 0; vt < VC; ++vt)
+  for (int a = 0; a < MAPS; ++a) {
+    const size_t row = (((size_t)z * total_q + tok) * H + head) * MAPS + a;
 #pragma unroll
-    for (int c = 0; c < 4; ++c) {
-      const int v = vt * 16 + 4 * lg + c;
-      if (v < dv) part_o[((size_t)z * total_q + tok) * H * dv + (size_t)head * dv + v] = o[vt][c];
+    for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+      for (int c = 0; c < 4; ++c) {
+        const int v = vt * 16 + 4 * lg + c;
+        if (v < dv) part_o[row * dv + v] = o[a][vt][c];
+      }
+    if (lg == 0) {
+      part_ml[row * 2] = m[a];
+      part_ml[row * 2 + 1] = lsum[a];
     }
-  if (lg == 0) {
-    float* ml = part_ml + (((size_t)z * total_q + tok) * H + head) * 2;
-    ml[0] = m;
-    ml[1] = lsum;
   }
 }
 
@@ -751,6 +849,52 @@ __global__ __launch_bounds__(64) void sink_merge_kernel(T* __restrict__ out, int
     for (int s = 0; s < splits; ++s)
       v = fmaf(part_o[((size_t)s * total_q + t) * H * dv + (size_t)h * dv + c], expf(part_ml[(((size_t)s * total_q + t) * H + h) * 2] - M), v);
     st(out + t * ld_out + (size_t)h * dv + c, v / den);
+  }
+}
+
+// The same for two maps: both joined over the ranges, then their difference, its norm, the factor and the gate.
+template <typename T>
+__global__ __launch_bounds__(64) void diff_merge_kernel(T* __restrict__ out, int64_t ld_out, const float* __restrict__ part_o,
+                                                        const float* __restrict__ part_ml, int total_q, int H, int dv, int splits, DiffOut df) {
+  const size_t t = blockIdx.x / H;
+  const int h = blockIdx.x % H;
+  float M[2] = {-INFINITY, -INFINITY}, f[2];
+  for (int s = 0; s < splits; ++s)
+#pragma unroll
+    for (int a = 0; a < 2; ++a) M[a] = fmaxf(M[a], part_ml[((((size_t)s * total_q + t) * H + h) * 2 + a) * 2]);
+#pragma unroll
+  for (int a = 0; a < 2; ++a) {
+    float den = 0.f;
+    for (int s = 0; s < splits; ++s) {
+      const float* ml = part_ml + ((((size_t)s * total_q + t) * H + h) * 2 + a) * 2;
+      den += ml[1] * expf(ml[0] - M[a]);
+    }
+    f[a] = (a == 0 ? 1.0f : -df.lam[0]) / den;
+  }
+  float o[4], ss = 0.f;  // dv <= 256
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = threadIdx.x + 64 * i;
+    o[i] = 0.f;
+    if (c < dv) {
+      for (int s = 0; s < splits; ++s)
+#pragma unroll
+        for (int a = 0; a < 2; ++a) {
+          const size_t row = (((size_t)s * total_q + t) * H + h) * 2 + a;
+          o[i] = fmaf(part_o[row * dv + c], f[a] * expf(part_ml[row * 2] - M[a]), o[i]);
+        }
+      ss = fmaf(o[i], o[i], ss);
+    }
+  }
+  const float n = df.post / sqrtf(wave_sum(ss) / (float)dv + df.eps);
+  const T* gate = cp<T>(df.gate);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int c = threadIdx.x + 64 * i;
+    if (c < dv) {
+      const float gz = gate ? sigmoidf_(ld(gate + t * df.ld_gate + (size_t)h * dv + c)) : 1.f;
+      st(out + t * ld_out + (size_t)h * dv + c, o[i] * n * gz);
+    }
   }
 }
 
@@ -959,21 +1103,50 @@ int msgl_mix_selective_scan(void* out, const void* x, int64_t ld_x, const void* 
   return MSGL_MIX_EINVAL;
 }
 
-int msgl_mix_sink_attn_workspace_floats(int total_q, int H, int dv, int splits) { return splits > 1 ? total_q * H * (dv + 2) * splits : 0; }
+// both forms of the attention: MAPS = 1 with an optional sink, MAPS = 2 the difference of two maps
+namespace {
 
-int msgl_mix_sink_attn(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table,
-                       int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G,
-                       int d, int dv, float scale, int window, const float* sink, int dtype, int splits, float* workspace, void* stream) {
+template <int KC, int VC, int MAPS>
+int sink_mfma_launch(dim3 grid, hipStream_t s, bf16_t* out, int64_t ld_out, float* part_o, float* part_ml, const float* q, const bf16_t* k_cache,
+                     const bf16_t* v_cache, const int* table, int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q,
+                     int batch, int total_q, int H, int G, int d, int dv, float scale, int window, int keep, const float* sink, DiffOut df,
+                     int QT, int HB, int splits) {
+  const size_t lds = (size_t)kNKT * ((MAPS * KC * 32 + 8) + (VC * 16 + 8)) * sizeof(uint16_t);
+  const int kvec = (((uintptr_t)k_cache & 15u) == 0 && d % 8 == 0) ? 1 : 0, vvec = (((uintptr_t)v_cache & 15u) == 0 && dv % 8 == 0) ? 1 : 0;
+  MIX_REQUIRE(ensure_lds((const void*)sink_attn_mfma_kernel<KC, VC, MAPS>, lds) == 0, "sink_attn: LDS request refused");
+  hipLaunchKernelGGL((sink_attn_mfma_kernel<KC, VC, MAPS>), grid, dim3(256), lds, s, out, ld_out, part_o, part_ml, q, k_cache, v_cache, table,
+                     table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d, dv, scale, window, keep, sink, df, QT, HB, splits, kvec,
+                     vvec);
+  MIX_LAUNCHED("sink_attn (matrix cores)");
+  return MSGL_MIX_OK;
+}
+
+template <typename T, int MAPS>
+int sink_merge_launch(hipStream_t s, T* out, int64_t ld_out, const float* part_o, const float* part_ml, int total_q, int H, int dv, int splits,
+                      const float* sink, DiffOut df) {
+  if (splits <= 1) return MSGL_MIX_OK;
+  if constexpr (MAPS == 1) {
+    hipLaunchKernelGGL(sink_merge_kernel<T>, dim3(total_q * H), dim3(64), 0, s, out, ld_out, part_o, part_ml, total_q, H, dv, splits, sink);
+  } else {
+    hipLaunchKernelGGL(diff_merge_kernel<T>, dim3(total_q * H), dim3(64), 0, s, out, ld_out, part_o, part_ml, total_q, H, dv, splits, df);
+  }
+  MIX_LAUNCHED("sink_attn merge");
+  return MSGL_MIX_OK;
+}
+
+template <int MAPS>
+int sink_attn_any(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table, int64_t table_stride,
+                  const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G, int d, int dv, float scale,
+                  int window, int keep, const float* sink, DiffOut df, int dtype, int splits, float* workspace, hipStream_t s) {
   MIX_REQUIRE(out && q && k_cache && v_cache && table && req_rows && seq_lens && cu_q && dtype_ok(dtype), "sink_attn: null pointer / dtype");
-  MIX_REQUIRE(batch >= 1 && total_q >= 0 && H >= 1 && G >= 1 && H % G == 0 && d >= 1 && dv >= 1 && dv <= 16 * kSinkMaxC &&
+  MIX_REQUIRE(batch >= 1 && total_q >= 0 && H >= 1 && G >= 1 && H % G == 0 && d >= 1 && dv >= 1 && dv <= 16 * kSinkMaxC && keep >= 0 &&
                   ld_out >= (int64_t)H * dv,
               "sink_attn: bad sizes H %d G %d d %d dv %d", H, G, d, dv);
   MIX_REQUIRE(splits >= 1 && splits <= 1024 && (splits == 1 || workspace), "sink_attn: %d splits need a workspace", splits);
   if (total_q == 0) return MSGL_MIX_OK;
   const int rep = H / G;
-  hipStream_t s = static_cast<hipStream_t>(stream);
   float* part_o = workspace;
-  float* part_ml = workspace ? workspace + (size_t)splits * total_q * H * dv : nullptr;
+  float* part_ml = workspace ? workspace + (size_t)splits * total_q * H * MAPS * dv : nullptr;
   if (dtype == MSGL_MIX_BF16 && d <= 256 && dv <= 256) {
     // matrix-core kernel: the smallest (KC, VC) instance that holds d <= 32 KC and dv <= 16 VC
     int HBm = 1;
@@ -982,47 +1155,65 @@ int msgl_mix_sink_attn(void* out, int64_t ld_out, const float* q, const void* k_
     const int groups_m = (total_q + QTm - 1) / QTm + batch;
     MIX_REQUIRE((int64_t)G * hbl <= 65535, "sink_attn: too many heads");
     const dim3 grid(groups_m, G * hbl, splits);
-    const int kvec = (((uintptr_t)k_cache & 15u) == 0 && d % 8 == 0) ? 1 : 0, vvec = (((uintptr_t)v_cache & 15u) == 0 && dv % 8 == 0) ? 1 : 0;
-#define SINK_CASE(KC, VC)                                                                                                                 \
-  if (d <= KC * 32 && dv <= VC * 16) {                                                                                                    \
-    const size_t lds_m = (size_t)kNKT * ((KC * 32 + 8) + (VC * 16 + 8)) * sizeof(uint16_t);                                               \
-    MIX_REQUIRE(ensure_lds((const void*)sink_attn_mfma_kernel<KC, VC>, lds_m) == 0, "sink_attn: LDS request refused");                    \
-    hipLaunchKernelGGL((sink_attn_mfma_kernel<KC, VC>), grid, dim3(256), lds_m, s, mp<bf16_t>(out), ld_out, part_o, part_ml, q,           \
-                       cp<bf16_t>(k_cache), cp<bf16_t>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d,  \
-                       dv, scale, window, sink, QTm, HBm, splits, kvec, vvec);                                                            \
-    MIX_LAUNCHED("sink_attn (matrix cores)");                                                                                             \
-    if (splits > 1) {                                                                                                                     \
-      hipLaunchKernelGGL(sink_merge_kernel<bf16_t>, dim3(total_q * H), dim3(64), 0, s, mp<bf16_t>(out), ld_out, part_o, part_ml, total_q, \
-                         H, dv, splits, sink);                                                                                            \
-      MIX_LAUNCHED("sink_attn merge");                                                                                                    \
-    }                                                                                                                                     \
-    return MSGL_MIX_OK;                                                                                                                   \
+#define SINK_CASE(KC, VC)                                                                                                                  \
+  if (d <= KC * 32 && dv <= VC * 16) {                                                                                                     \
+    const int rc = sink_mfma_launch<KC, VC, MAPS>(grid, s, mp<bf16_t>(out), ld_out, part_o, part_ml, q, cp<bf16_t>(k_cache),               \
+                                                  cp<bf16_t>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H,   \
+                                                  G, d, dv, scale, window, keep, sink, df, QTm, HBm, splits);                              \
+    return rc ? rc : sink_merge_launch<bf16_t, MAPS>(s, mp<bf16_t>(out), ld_out, part_o, part_ml, total_q, H, dv, splits, sink, df);       \
   }
-    SINK_CASE(2, 4)
-    SINK_CASE(3, 6)
-    SINK_CASE(4, 8)
-    SINK_CASE(6, 12)
-    SINK_CASE(8, 16)
+    if constexpr (MAPS == 1) {
+      SINK_CASE(2, 4)
+      SINK_CASE(3, 6)
+      SINK_CASE(4, 8)
+      SINK_CASE(6, 12)
+      SINK_CASE(8, 16)
+    } else {  // the values of two maps are usually twice as wide as one map's keys; maps above 128 take the plain kernel
+      SINK_CASE(1, 4)
+      SINK_CASE(2, 4)
+      SINK_CASE(2, 8)
+      SINK_CASE(4, 8)
+      SINK_CASE(4, 16)
+    }
 #undef SINK_CASE
   }
   int HB = 1;
   while (HB * 2 <= rep && HB * 2 <= kSinkRows) HB *= 2;
   const int QT = kSinkRows / HB, hblocks = (rep + HB - 1) / HB;
   int KT = 64;
-  auto need = [&](int kt) { return (size_t)((kSinkRows + kt) * (d + 1) + kt * (dv + 1) + kSinkRows * kt) * sizeof(float); };
+  auto need = [&](int kt) { return (size_t)((kSinkRows + kt) * (MAPS * d + 1) + kt * (dv + 1) + MAPS * kSinkRows * kt) * sizeof(float); };
   while (KT > 8 && need(KT) > 160 * 1024) KT >>= 1;
   const size_t lds = need(KT);
   MIX_REQUIRE(lds <= 160 * 1024, "sink_attn: heads of %d / %d do not fit LDS", d, dv);
   const int groups = (total_q + QT - 1) / QT + batch;  // every request may end with one partial group
   MIX_REQUIRE((int64_t)G * hblocks <= 65535, "sink_attn: too many heads");
-  DISPATCH_T(dtype, MIX_REQUIRE(ensure_lds((const void*)sink_attn_kernel<T>, lds) == 0, "sink_attn: LDS request refused");
-             hipLaunchKernelGGL(sink_attn_kernel<T>, dim3(groups, G * hblocks, splits), dim3(256), lds, s, mp<T>(out), ld_out, part_o,
+  DISPATCH_T(dtype, MIX_REQUIRE((ensure_lds((const void*)sink_attn_kernel<T, MAPS>, lds) == 0), "sink_attn: LDS request refused");
+             hipLaunchKernelGGL((sink_attn_kernel<T, MAPS>), dim3(groups, G * hblocks, splits), dim3(256), lds, s, mp<T>(out), ld_out, part_o,
                                 part_ml, q, cp<T>(k_cache), cp<T>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H,
-                                G, d, dv, scale, window, sink, QT, HB, KT, splits);
-             if (splits > 1) hipLaunchKernelGGL(sink_merge_kernel<T>, dim3(total_q * H), dim3(64), 0, s, mp<T>(out), ld_out, part_o, part_ml,
-                                                total_q, H, dv, splits, sink);)
-  MIX_LAUNCHED("sink_attn");
-  return MSGL_MIX_OK;
+                                G, d, dv, scale, window, keep, sink, df, QT, HB, KT, splits);
+             MIX_LAUNCHED("sink_attn");
+             return (sink_merge_launch<T, MAPS>(s, mp<T>(out), ld_out, part_o, part_ml, total_q, H, dv, splits, sink, df));)
+}
+
+}  // namespace
+
+int msgl_mix_sink_attn_workspace_floats(int total_q, int H, int dv, int splits) { return splits > 1 ? total_q * H * (dv + 2) * splits : 0; }
+
+int msgl_mix_sink_attn(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table,
+                       int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G,
+                       int d, int dv, float scale, int window, int keep, const float* sink, int dtype, int splits, float* workspace,
+                       void* stream) {
+  return sink_attn_any<1>(out, ld_out, q, k_cache, v_cache, table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d, dv, scale,
+                          window, keep, sink, DiffOut{nullptr, nullptr, 0, 1.f, 0.f}, dtype, splits, workspace, static_cast<hipStream_t>(stream));
+}
+
+int msgl_mix_diff_attn(void* out, int64_t ld_out, const float* q, const void* k_cache, const void* v_cache, const int* table,
+                       int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G,
+                       int d, int dv, float scale, int window, int keep, const float* lam, float post, float eps, const void* gate,
+                       int64_t ld_gate, int dtype, int splits, float* workspace, void* stream) {
+  MIX_REQUIRE(lam && (!gate || ld_gate >= (int64_t)H * dv), "diff_attn: no weight of the second map, or gate rows too short");
+  return sink_attn_any<2>(out, ld_out, q, k_cache, v_cache, table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d, dv, scale,
+                          window, keep, nullptr, DiffOut{lam, gate, ld_gate, post, eps}, dtype, splits, workspace, static_cast<hipStream_t>(stream));
 }
 
 int msgl_mix_route_sigmoid(int* ids, float* wts, const float* z, int tokens, int E, int top, void* stream) {

@@ -74,7 +74,21 @@ feed-forward       W_down (silu(W_gate h) * (W_up h)), or routed experts of that
                    largest chosen, a chosen expert runs on score * h (the weight enters BEFORE the expert, so the choices' outputs are
                    summed as they are), plus a shared expert that every token runs.
 
-Kernels: csrc/seqmix.hip, csrc/mix_delta.hip, csrc/mix_par.hip and csrc/mix_scan.hip through mixops.py; plain projections through the library GEMM
+A fifth scheme, `streams` (the Nagezen design): s residual streams instead of one, an element-wise squashing in the place of every norm:
+
+stream             all x_k = embed[token];  per sublayer  u = sum_k in[k] x_k,  y = sublayer(n(u)),  x_t <- sum_k mix[k, t] x_k + out[t] y
+                   (all streams at once from the old ones);  n(u) = tanh(alpha u) w + b, no statistic of the row.  Output: n of the
+                   streams' sum, head matrix, times a logit scale.  The streams are one fp32 tensor [tokens, s, W].
+retention          q and k turn by position, k d^-1/2;  S <- decay_h S + k v^T, o = S^T q;  heads divided by their root mean square,
+                   gated by silu(W_g h).
+gla                the same with a decay per key channel, sigmoid(W_a2 W_a1 h + bias)^(1 / tau), q d^-1/2 and a weighted head norm.
+diff_attention     two softmax maps over the same values per head (q and k hold [map 1 | map 2], projection biases, weighted RMS norm of
+                   every map row, rotation), o = a1 - lambda a2 with one learned lambda per layer, unit RMS per head times
+                   (1 - diff), gated by sigmoid(W_g h).  Token i sees the last `window` keys and the first `keep_first` of the
+                   sequence.  Cached per token: k [G 2 d] and v [G dv].
+feed-forward       W_down of  g sigmoid(1.702 g) (u + 1),  g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit).
+
+Kernels: csrc/seqmix.hip, csrc/mix_delta.hip, csrc/mix_par.hip, csrc/mix_scan.hip and csrc/mix_streams.hip through mixops.py; plain projections through the library GEMM
 (mixops.linear).
 """
 from __future__ import annotations
@@ -109,12 +123,19 @@ class DenseFfSpec:
     act: str = "poly_norm"          # "poly_norm": c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 with N = divide a row by its root mean square;
                                     # "xielu": softplus(p) z^2 + z / 2 above zero, (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 below
                                     # "silu_gate": W_down (silu(W_gate h) * (W_up h))
+                                    # "clamp_gate": W_down (g sigmoid(slope g) (u + 1)), g = min(W_gate h, limit), u = W_up h within +-limit
+    limit: float = 0.0              # clamp_gate
+    slope: float = 1.702
+
+    @property
+    def gated(self) -> bool:
+        return self.act in ("silu_gate", "clamp_gate")
 
 
 @dataclass(frozen=True)
 class LayerSpec:
     kind: str                       # "latent_attention" | "lightning" | "attention" | "delta" | "channel_delta" | "parallel" |
-                                    # "sink_attention" | "mamba1";
+                                    # "sink_attention" | "mamba1" | "retention" | "gla" | "diff_attention";
                                     # inside a "parallel" pair: "sigmoid_attention" | "state_space"
     heads: int
     dim: int                        # unrotated query/key size per head (lightning: query/key size)
@@ -145,12 +166,16 @@ class LayerSpec:
     out_gate: bool = False          # latent attention: the concatenated heads are multiplied by sigmoid(W_g h)
     v_norm: bool = False            # sink attention: every value head is divided by its root mean square before it is cached
     dt_rank: int = 0                # mamba1: inner size of the two-step step-size projection
+    maps: int = 1                   # diff_attention: 2, the softmax maps whose difference a head is
+    keep_first: int = 0             # diff_attention: the first so many keys of a sequence stay visible behind the window
+    diff: float = 0.0               # diff_attention: constant part of the second map's weight; the output is scaled by 1 - diff
+    tau: float = 1.0                # gla: a decay is the tau-th root of a sigmoid
     # state space: heads x vdim = inner size, dim = state size per head, kv_heads = groups of B / C, conv = taps
     # mamba1: heads = 1, vdim = inner size (channels), dim = state size per channel, conv = taps
 
     @property
     def recurrent(self) -> bool:
-        return self.kind in ("lightning", "delta", "channel_delta", "state_space", "mamba1") or \
+        return self.kind in ("lightning", "delta", "channel_delta", "state_space", "mamba1", "retention", "gla") or \
             (self.kind == "parallel" and (self.left.recurrent or self.right.recurrent))
 
 
@@ -176,6 +201,9 @@ class HybridConfig:
     residual_mult: float = 1.0
     logit_softcap: float = 0.0      # logits <- cap tanh(logits / cap); 0 = none
     loop: Optional[Tuple[int, int, int]] = None   # (start, stop, times): layers start .. stop - 1 run `times` times in a row
+    # "streams": several residual streams joined by small matrices around every sublayer, tanh in the place of norms, own head
+    streams: int = 1
+    logit_scale: float = 1.0        # logits <- scale * head x
 
     @property
     def num_layers(self) -> int:
@@ -383,6 +411,48 @@ def piladra_config(cfg: Dict[str, Any], name: str = "Piladra") -> HybridConfig:
                         residual_mult=float(cfg.get("residual_mult", 1.0)), logit_softcap=float(cfg.get("logit_softcap") or 0.0), loop=lp)
 
 
+def nagezen_config(cfg: Dict[str, Any], shapes: Optional[Dict[str, Tuple[int, ...]]] = None, name: str = "Nagezen") -> HybridConfig:
+    """config.json of a Nagezen model -> HybridConfig.  `shapes` (tensor name -> shape, from the checkpoint's header) gives the inner
+    size of a gla layer's two-step decay projection, which config.json leaves to the tensors."""
+    shapes = shapes or {}
+    layers: List[LayerSpec] = []
+    for i, entry in enumerate(cfg["layers"]):
+        m, kind, mlp = entry["mixer"], entry["type"], entry.get("mlp")
+        ff = None
+        if mlp is not None:
+            if mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+            ff = DenseFfSpec(ff=int(mlp["ff"]), act="clamp_gate", limit=float(mlp["limit"]))
+        H, d, dv = int(m["heads"]), int(m["dim"]), int(m["vdim"])
+        dims, base = _rot(m, 0)
+        if dims % 2 or dims > d:
+            raise ValueError(f"layer {i}: a rotation of {dims} entries in heads of {d}")
+        if kind == "retention":
+            decay = tuple(float(x) for x in m["decay"])
+            if len(decay) != H:
+                raise ValueError(f"layer {i}: {len(decay)} decays for {H} heads")
+            layers.append(LayerSpec(kind="retention", heads=H, dim=d, vdim=dv, decay=decay, rot_dims=dims, rot_base=base, mlp=ff))
+        elif kind == "gla":
+            rank = int(shapes.get(f"l{i}.mix.a1", (16,))[0])
+            layers.append(LayerSpec(kind="gla", heads=H, dim=d, vdim=dv, tau=float(m["tau"]), decay_rank=rank, mlp=ff))
+        elif kind == "attention":
+            G, mask = int(m.get("kv_heads", H)), m.get("mask") or {}
+            sc = (m.get("rot") or {}).get("scaling")
+            if H % G:
+                raise ValueError(f"layer {i}: {H} heads over {G} key heads")
+            layers.append(LayerSpec(kind="diff_attention", heads=H, kv_heads=G, dim=d, vdim=dv, scale=float(m["scale"]), maps=2,
+                                    window=int(mask.get("size", 0)), keep_first=int(mask.get("keep_first", 0)), diff=float(m["diff"]),
+                                    rot_dims=dims, rot_base=base,
+                                    rot_scaling=None if not sc else tuple(sorted((k, float(v)) for k, v in sc.items())), out_gate=True, mlp=ff))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+    streams = int(cfg.get("streams", 1))
+    if not 1 <= streams <= 16:
+        raise ValueError(f"{streams} residual streams")
+    return HybridConfig(vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]), layers=tuple(layers), rms_norm_eps=float(cfg["norm"]["eps"]),
+                        name=name, residual="streams", streams=streams, logit_scale=float(cfg.get("logit_scale", 1.0)))
+
+
 def wavelength_scaled_rotary_table(dims: int, base: float, scaling: Optional[Dict[str, float]], max_position: int, device) -> torch.Tensor:
     """fp32 [max_position, dims] = cos | sin of position * f_i, f_i = base^(-2i / dims) rescaled by wavelength l = 2 pi / f: kept where
     l < original / high, divided by `factor` where l > original / low, blended linearly in original / l between; float64, rounded once."""
@@ -418,12 +488,32 @@ class _Layer:
     __slots__ = ("spec", "w_in", "o", "norm1", "norm2", "uk_t", "uv", "c_norm", "cos_sin", "out_norm", "decay", "router",
                  "bias", "up", "down", "talk", "lam", "taps", "rate", "dt_bias", "a2", "g2", "act", "depth_w",
                  "sink", "ls1", "ls2", "shift", "in_bias", "out_bias", "pb", "skip", "conv_b", "sum_bias", "canon1", "canon2", "w_x", "w_dt",
-                 "sh_up", "sh_down")
+                 "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k", "lam_now", "sq1", "sq2", "hc1", "hc2")
 
     def __init__(self, spec: LayerSpec) -> None:
         self.spec = spec
         for k in self.__slots__[1:]:
             setattr(self, k, None)
+
+
+class _Squash:
+    """tanh(alpha u) w + b, element by element: what stands in the place of a norm; alpha is fp32 [1] on the device."""
+    __slots__ = ("w", "b", "alpha")
+
+    def __init__(self, w: torch.Tensor, b: torch.Tensor, alpha: torch.Tensor) -> None:
+        self.w, self.b, self.alpha = w, b, alpha
+
+    @property
+    def parts(self):
+        return self.w, self.b, self.alpha
+
+
+class _Junction:
+    """How one sublayer reads from the residual streams and writes to them: read [s], out [s], mix [s (from), s (to)], fp32."""
+    __slots__ = ("read", "out", "mix")
+
+    def __init__(self, read: torch.Tensor, out: torch.Tensor, mix: torch.Tensor) -> None:
+        self.read, self.out, self.mix = read, out, mix
 
 
 class HybridDecoder:
@@ -448,9 +538,11 @@ class HybridDecoder:
         self.pre_norm = cfg.residual == "pre_norm_depth"
         self.parallel = cfg.residual == "parallel_shift"
         self.conv_stream = cfg.residual == "pre_norm_conv"
+        self.multi = cfg.residual == "streams"
+        self.final_squash: Optional[_Squash] = None
         self.embed_norm = self.head = self.pair_table = self.loop_step = None
         self.embed = w(cfg.vocab_size, W, std=1.0)
-        self.final_norm = w(W, std=0.1)
+        self.final_norm = None if self.multi else w(W, std=0.1)
         self.layers: List[_Layer] = []
         tables: Dict[tuple, torch.Tensor] = {}
 
@@ -463,10 +555,22 @@ class HybridDecoder:
                 tables[key] = plain_rotary_table(dims, base, self.max_position, device)
             return tables[key]
 
+        def squash():
+            return _Squash((1.0 + w(W, std=0.1).float()).to(dtype), w(W, std=0.1), f32(1, std=0.1, mean=0.6))
+
+        def junction():
+            n = cfg.streams
+            return _Junction(f32(n, std=0.2, mean=1.0 / n), f32(n, std=0.3, mean=0.8),
+                             f32(n, n, std=0.15) + 0.8 * torch.eye(n, dtype=torch.float32, device=device))
+
         for spec in cfg.layers:
             L = _Layer(spec)
+            if self.multi:
+                L.sq1, L.hc1 = squash(), junction()
+                if spec.mlp is not None:
+                    L.sq2, L.hc2 = squash(), junction()
             H, d, dv = spec.heads, spec.dim, spec.vdim
-            L.norm1 = w(W, std=0.1)
+            L.norm1 = None if self.multi else w(W, std=0.1)
             if self.parallel:
                 L.norm1, L.ls1, L.ls2 = f32(W, std=0.1), f32(W, std=0.2, mean=1.0), f32(W, std=0.2, mean=1.0)
                 L.shift = f32(W, std=0.2, mean=0.5) if cfg.token_shift else None
@@ -486,6 +590,29 @@ class HybridDecoder:
                 # one output projection over the row [attention heads | state-space channels]
                 L.o = w(W, H * dv + inner, std=(H * dv + inner) ** -0.5)
                 L.out_bias = f32(W, std=0.1)
+            elif spec.kind in ("retention", "gla"):
+                L.w_in = w(2 * H * d + 2 * H * dv + spec.decay_rank, W, std=W ** -0.5)  # q | k | v | gate (| decay input)
+                L.o = w(W, H * dv, std=(H * dv) ** -0.5)
+                if spec.kind == "gla":
+                    L.a2 = w(H * d, spec.decay_rank, std=spec.decay_rank ** -0.5)
+                    L.dt_bias = f32(H * d, std=0.5, mean=1.0)
+                    L.out_norm = (1.0 + w(dv, std=0.1).float()).to(dtype)
+                else:
+                    L.decay = torch.tensor(spec.decay, dtype=torch.float32, device=device)
+                    L.cos_sin = plain_table(spec.rot_dims, spec.rot_base) if spec.rot_dims else None
+            elif spec.kind == "diff_attention":
+                G, n = spec.kv_heads, (H + spec.kv_heads) * spec.maps * d + spec.kv_heads * dv
+                L.w_in = w(n + H * dv, W, std=W ** -0.5)  # q | k | v | gate
+                L.in_bias = f32(n, std=0.1)
+                L.q_norm, L.k_norm = (1.0 + w(d, std=0.1).float()).to(dtype), (1.0 + w(d, std=0.1).float()).to(dtype)
+                L.lam_q, L.lam_k = f32(spec.maps, d, std=0.1), f32(spec.maps, d, std=0.1)
+                L.lam_now = f32(1)
+                L.o = w(W, H * dv, std=(H * dv) ** -0.5)
+                if spec.rot_dims:
+                    key = (spec.rot_dims, spec.rot_base, spec.rot_scaling)
+                    if key not in tables:
+                        tables[key] = rotary_table(spec, self.max_position, device)
+                    L.cos_sin = tables[key]
             elif spec.kind == "mamba1":
                 inner, N, dr = spec.vdim, spec.dim, spec.dt_rank
                 L.w_in = w(2 * inner, W, std=W ** -0.5)           # x | z
@@ -554,10 +681,10 @@ class HybridDecoder:
                 L.up = w(m.experts, (2 if m.gated else 1) * m.ff, W, std=W ** -0.5)  # gated: every expert's gate rows, then its up rows
                 L.down = w(m.experts, W, m.ff, std=m.ff ** -0.5)
             elif isinstance(m, DenseFfSpec):
-                L.norm2 = None if self.parallel else w(W, std=0.1)
-                L.up = w((2 if m.act == "silu_gate" else 1) * m.ff, W, std=W ** -0.5)  # silu_gate: the gate rows, then the up rows
+                L.norm2 = None if self.parallel or self.multi else w(W, std=0.1)
+                L.up = w((2 if m.gated else 1) * m.ff, W, std=W ** -0.5)  # gated: the gate rows, then the up rows
                 L.down = w(W, m.ff, std=m.ff ** -0.5)
-                L.act = torch.tensor([0.3, -0.4] if m.act == "xielu" else [1.0, 0.3, 0.1, 0.01], dtype=torch.float32, device=device)
+                L.act = None if m.gated else torch.tensor([0.3, -0.4] if m.act == "xielu" else [1.0, 0.3, 0.1, 0.01], dtype=torch.float32, device=device)
             if isinstance(m, MoeSpec) and m.shared_ff:
                 L.sh_up = w(2 * m.shared_ff, W, std=W ** -0.5)
                 L.sh_down = w(W, m.shared_ff, std=m.shared_ff ** -0.5)
@@ -581,6 +708,10 @@ class HybridDecoder:
             self.head = w(cfg.vocab_size, W, std=W ** -0.5)
             if cfg.loop is not None:
                 self.loop_step = f32(cfg.loop[2], W, std=0.3)
+        if self.multi:
+            self.final_squash = squash()
+            self.head = w(cfg.vocab_size, W, std=W ** -0.5)
+            self._derive()
         if self.parallel:
             self.final_norm = f32(W, std=0.1)
             self.head = w(cfg.vocab_size, W, std=W ** -0.5)
@@ -591,24 +722,35 @@ class HybridDecoder:
     # ------------------------------------------------------------------ weights
     def _derive(self) -> None:
         """What the kernels read that is a function of loaded tensors: a pair layer's output bias as it enters the residual sum
-        (the attention's projection bias times the attention's scale times the layer scale of the mixer)."""
+        (the attention's projection bias times the attention's scale times the layer scale of the mixer); the weight of a differential
+        attention's second map.  Written in place: a captured graph reads the tensor's address."""
         for L in self.layers:
             if L.spec.kind == "parallel":
                 L.sum_bias = (L.out_bias * L.spec.left_scale * L.ls1).contiguous()
+            if L.spec.kind == "diff_attention":
+                e = torch.exp((L.lam_q.double() * L.lam_k.double()).sum(dim=1))
+                L.lam_now.copy_((e[0] - e[1] + L.spec.diff).reshape(1))
 
     def _tensors(self):
         yield self.embed
-        yield self.final_norm
-        for t in (self.embed_norm, self.head, self.pair_table, self.loop_step):
+        for t in (self.final_norm, self.embed_norm, self.head, self.pair_table, self.loop_step):
             if t is not None:
                 yield t
         for L in self.layers:
             for k in ("w_in", "o", "norm1", "norm2", "uk_t", "uv", "c_norm", "out_norm", "router", "bias", "up", "down", "talk", "lam",
                       "taps", "rate", "dt_bias", "a2", "g2", "act", "depth_w", "sink", "ls1", "ls2", "shift", "in_bias", "out_bias", "pb",
-                      "skip", "conv_b", "canon1", "canon2", "w_x", "w_dt", "sh_up", "sh_down"):
+                      "skip", "conv_b", "canon1", "canon2", "w_x", "w_dt", "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k"):
                 t = getattr(L, k)
                 if t is not None:
                     yield t
+            for k in ("sq1", "sq2"):
+                if getattr(L, k) is not None:
+                    yield from getattr(L, k).parts
+            for k in ("hc1", "hc2"):
+                if getattr(L, k) is not None:
+                    yield from (getattr(L, k).read, getattr(L, k).out, getattr(L, k).mix)
+        if self.final_squash is not None:
+            yield from self.final_squash.parts
 
     def weight_bytes(self) -> int:
         return sum(t.numel() * t.element_size() for t in self._tensors())
@@ -627,8 +769,22 @@ class HybridDecoder:
                 raise ValueError(f"checkpoint tensor of shape {tuple(src.shape)} where the config implies {tuple(dst.shape)}")
             dst.copy_(src.to(device=self.device, dtype=torch.float32))  # rounds to the destination's dtype (fp32 tensors stay fp32)
 
+        def put_squash(sq: _Squash, name: str) -> None:
+            put(sq.w, state[name])
+            put(sq.b, state[name + ".b"])
+            put(sq.alpha, state[name + ".alpha"].reshape(1))
+
+        def put_junction(hc: _Junction, name: str) -> None:
+            put(hc.read, state[name + ".in"])
+            put(hc.out, state[name + ".out"])
+            put(hc.mix, state[name + ".mix"])
+
         put(self.embed, state["embed"])
-        put(self.final_norm, state["final.norm"])
+        if self.multi:
+            put_squash(self.final_squash, "final.norm")
+            put(self.head, state["head"])
+        else:
+            put(self.final_norm, state["final.norm"])
         if self.pre_norm:
             put(self.embed_norm, state["embed.norm"])
             put(self.head, state["head"])
@@ -643,7 +799,14 @@ class HybridDecoder:
         for i, L in enumerate(self.layers):
             s, p = L.spec, f"l{i}.mix."
             H, d, dv = s.heads, s.dim, s.vdim
-            put(L.norm1, state[f"l{i}.norm1"])
+            if self.multi:
+                put_squash(L.sq1, f"l{i}.norm1")
+                put_junction(L.hc1, f"l{i}.hc1")
+                if s.mlp is not None:
+                    put_squash(L.sq2, f"l{i}.norm2")
+                    put_junction(L.hc2, f"l{i}.hc2")
+            else:
+                put(L.norm1, state[f"l{i}.norm1"])
             if L.canon1 is not None:
                 put(L.canon1, state[f"l{i}.canon1"])
             if L.canon2 is not None:
@@ -671,6 +834,19 @@ class HybridDecoder:
                 put(L.out_norm, state[b + "norm"])
                 put(L.o, torch.cat([state[a + "o"], state[b + "o"]], dim=1))
                 put(L.out_bias, state[a + "o.b"])
+            elif s.kind in ("retention", "gla"):
+                put(L.w_in, torch.cat([state[p + n] for n in ("q", "k", "v", "g") + (("a1",) if s.kind == "gla" else ())], dim=0))
+                if s.kind == "gla":
+                    put(L.a2, state[p + "a2"])
+                    put(L.dt_bias, state[p + "a2.b"])
+                    put(L.out_norm, state[p + "norm"])
+            elif s.kind == "diff_attention":
+                put(L.w_in, torch.cat([state[p + n] for n in ("q", "k", "v", "g")], dim=0))
+                put(L.in_bias, torch.cat([state[p + n + ".b"] for n in ("q", "k", "v")], dim=0))
+                put(L.q_norm, state[p + "q.norm"])
+                put(L.k_norm, state[p + "k.norm"])
+                put(L.lam_q, torch.stack([state[p + "lq1"], state[p + "lq2"]]))
+                put(L.lam_k, torch.stack([state[p + "lk1"], state[p + "lk2"]]))
             elif s.kind == "mamba1":
                 put(L.w_in, state[p + "in"])
                 put(L.taps, state[p + "conv"])
@@ -708,12 +884,14 @@ class HybridDecoder:
                 put(L.out_norm, state[p + "norm"])
             if s.kind != "parallel":
                 put(L.o, state[p + "o"])
-            if s.mlp is None and f"l{i}.norm2" in state and not self.pre_norm and not self.parallel and not self.conv_stream:  # no feed-forward, but a second norm
+            if s.mlp is None and f"l{i}.norm2" in state and not self.pre_norm and not self.parallel and not self.conv_stream and \
+                    not self.multi:  # no feed-forward, but a second norm
                 L.norm2 = torch.empty_like(L.norm1)
                 put(L.norm2, state[f"l{i}.norm2"])
-            if isinstance(s.mlp, DenseFfSpec) and s.mlp.act == "silu_gate":
+            if isinstance(s.mlp, DenseFfSpec) and s.mlp.gated:
                 q = f"l{i}.mlp."
-                put(L.norm2, state[f"l{i}.norm2"])
+                if not self.multi:
+                    put(L.norm2, state[f"l{i}.norm2"])
                 put(L.up, torch.cat([state[q + "gate"], state[q + "up"]], dim=0))
                 put(L.down, state[q + "down"])
             elif isinstance(s.mlp, DenseFfSpec):
@@ -750,7 +928,12 @@ class HybridDecoder:
 
     def export_state(self) -> Dict[str, torch.Tensor]:
         """The inverse of load_state (checkpoint names, host tensors): what tests and tools hand to an independent implementation."""
-        out = {"embed": self.embed, "final.norm": self.final_norm}
+        out = {"embed": self.embed}
+        if self.multi:
+            out["head"] = self.head
+            out["final.norm"], out["final.norm.b"], out["final.norm.alpha"] = *self.final_squash.parts[:2], self.final_squash.alpha.reshape(())
+        else:
+            out["final.norm"] = self.final_norm
         if self.pre_norm:
             out["embed.norm"], out["head"] = self.embed_norm, self.head
         if self.parallel:
@@ -764,7 +947,13 @@ class HybridDecoder:
         for i, L in enumerate(self.layers):
             s, p = L.spec, f"l{i}.mix."
             H, d, dv = s.heads, s.dim, s.vdim
-            out[f"l{i}.norm1"] = L.norm1
+            for k, sq, hc in ((1, L.sq1, L.hc1), (2, L.sq2, L.hc2)):
+                if sq is not None:
+                    n, j = f"l{i}.norm{k}", f"l{i}.hc{k}"
+                    out[n], out[n + ".b"], out[n + ".alpha"] = sq.w, sq.b, sq.alpha.reshape(())
+                    out[j + ".in"], out[j + ".out"], out[j + ".mix"] = hc.read, hc.out, hc.mix
+            if not self.multi:
+                out[f"l{i}.norm1"] = L.norm1
             if L.canon1 is not None:
                 out[f"l{i}.canon1"] = L.canon1
             if L.canon2 is not None:
@@ -789,6 +978,22 @@ class HybridDecoder:
                 out[b + "A_log"], out[b + "D"], out[b + "norm"] = torch.log(-L.rate), L.skip, L.out_norm
                 out[a + "o"], out[b + "o"] = L.o[:, : H * dv], L.o[:, H * dv:]
                 out[a + "o.b"] = L.out_bias
+            elif s.kind in ("retention", "gla"):
+                names, cuts = ["q", "k", "v", "g"], [H * d, H * d, H * dv, H * dv]
+                if s.kind == "gla":
+                    names, cuts = names + ["a1"], cuts + [s.decay_rank]
+                    out[p + "a2"], out[p + "a2.b"], out[p + "norm"] = L.a2, L.dt_bias, L.out_norm
+                for n, t in zip(names, torch.split(L.w_in, cuts, dim=0)):
+                    out[p + n] = t
+            elif s.kind == "diff_attention":
+                cuts = [H * s.maps * d, s.kv_heads * s.maps * d, s.kv_heads * dv]
+                for n, t in zip(("q", "k", "v", "g"), torch.split(L.w_in, cuts + [H * dv], dim=0)):
+                    out[p + n] = t
+                for n, t in zip(("q", "k", "v"), torch.split(L.in_bias, cuts, dim=0)):
+                    out[p + n + ".b"] = t
+                out[p + "q.norm"], out[p + "k.norm"] = L.q_norm, L.k_norm
+                for a in range(s.maps):
+                    out[p + f"lq{a + 1}"], out[p + f"lk{a + 1}"] = L.lam_q[a], L.lam_k[a]
             elif s.kind == "mamba1":
                 out[p + "in"], out[p + "conv"], out[p + "conv.b"], out[p + "x"], out[p + "dt"] = L.w_in, L.taps, L.conv_b, L.w_x, L.w_dt
                 out[p + "dt.b"], out[p + "A_log"], out[p + "D"] = L.dt_bias, torch.log(-L.rate), L.skip
@@ -825,9 +1030,11 @@ class HybridDecoder:
                 out[p + "o"] = L.o
             if s.mlp is None and L.norm2 is not None:
                 out[f"l{i}.norm2"] = L.norm2
-            if isinstance(s.mlp, DenseFfSpec) and s.mlp.act == "silu_gate":
+            if isinstance(s.mlp, DenseFfSpec) and s.mlp.gated:
                 q = f"l{i}.mlp."
-                out[f"l{i}.norm2"], out[q + "gate"], out[q + "up"], out[q + "down"] = L.norm2, L.up[: s.mlp.ff], L.up[s.mlp.ff:], L.down
+                out[q + "gate"], out[q + "up"], out[q + "down"] = L.up[: s.mlp.ff], L.up[s.mlp.ff:], L.down
+                if not self.multi:
+                    out[f"l{i}.norm2"] = L.norm2
             elif isinstance(s.mlp, DenseFfSpec):
                 q = f"l{i}.mlp."
                 out[q + "up"], out[q + "down"], out[q + "act"] = L.up, L.down, L.act
@@ -984,6 +1191,73 @@ class HybridDecoder:
             mixops.commit_rows(kv.conv_in_states.view(2 * len(runs), -1, (n - 1) * W), staging.view(2 * len(runs), bs, (n - 1) * W), md.req_rows, bs,
                                md.cu_seqlens_q)
         return hf
+
+    def _decay_attention(self, i: int, L: _Layer, h: torch.Tensor, ctx: Any, batch: Any) -> torch.Tensor:
+        """Linear attention with decays (retention, gla): one projection (and the second step of the decays'), rotation, recurrence on
+        the request's fp32 state, head norm and gate in one launch, output projection."""
+        s, md = L.spec, batch.attn_metadata
+        H, d, dv = s.heads, s.dim, s.vdim
+        proj = mixops.linear(h, L.w_in)
+        q, k, v, gate = (proj[:, a: b] for a, b in ((0, H * d), (H * d, 2 * H * d), (2 * H * d, 2 * H * d + H * dv),
+                                                    (2 * H * d + H * dv, 2 * H * d + 2 * H * dv)))
+        if s.kind == "gla":
+            decays = dict(z=mixops.linear(proj[:, 2 * H * d + 2 * H * dv:], L.a2), z_bias=L.dt_bias, tau=s.tau, q_scale=d ** -0.5, weight=L.out_norm)
+        else:
+            decays = dict(decay=L.decay, k_scale=d ** -0.5, cos_sin=L.cos_sin, positions=batch.positions)
+        y = mixops.decay_attn(q, k, v, gate, ctx.kv_cache.state(i), md.cu_seqlens_q, md.seq_lens, md.req_rows, md.batch, self.cfg.rms_norm_eps,
+                              chunks=getattr(md, "decay_chunks", None), **decays)
+        return mixops.linear(y, L.o)
+
+    def _diff_attention(self, i: int, L: _Layer, h: torch.Tensor, ctx: Any, batch: Any) -> torch.Tensor:
+        """Difference of two softmax maps: projections (+ bias), weighted norm and rotation of every map row, cache rows; both maps, their
+        difference, the head norm and the gate in one launch (two when the keys are cut into ranges); output projection."""
+        s, md, kv, eps = L.spec, batch.attn_metadata, ctx.kv_cache, self.cfg.rms_norm_eps
+        T, H, G, d, dv, M = h.shape[0], s.heads, s.kv_heads, s.dim, s.vdim, s.maps
+        proj = mixops.linear(h, L.w_in)
+        kc, vc = kv.kv_rows(i)
+        q = mixops.qk_prep(proj, L.in_bias, kc, vc, batch.out_loc, batch.positions, L.cos_sin, eps, H * M, G * M, d, dv, interleaved=False,
+                           unit=False, norm_w=(L.q_norm, L.k_norm), value_heads=G)
+        o = torch.empty((T, H * dv), dtype=self.dtype, device=h.device)
+        splits = mixops.sink_attn_splits(md.batch, T, H, G, s.window, md.max_seqlen_k, s.keep_first) if md.max_seqlen_q <= 16 else 1
+        mixops.diff_attn(o, q, kc, vc, ctx.page_table, md.req_rows, md.seq_lens, md.cu_seqlens_q, md.batch, H, G, d, dv, s.scale, s.window,
+                         s.keep_first, L.lam_now, 1.0 - s.diff, eps, gate=proj[:, L.in_bias.shape[0]:], splits=splits)
+        return mixops.linear(o, L.o)
+
+    def _forward_streams(self, ctx: Any, batch: Any, layer_outputs: Optional[list]) -> torch.Tensor:
+        """Several residual streams -> the rows in front of the LM head [tokens, W].  One `stream_norm` launch closes a sublayer (all
+        streams at once from the old ones) and opens the next (its read weights and squashing); the streams are updated in place."""
+        cfg = self.cfg
+        T, W, n, dev = batch.input_ids.shape[0], cfg.hidden_size, cfg.streams, self.device
+        x0 = mixops.embed_scaled(self.embed, batch.input_ids, 1.0)
+        xs = torch.empty((T, n, W), dtype=torch.float32, device=dev)
+        subs = []  # (layer, sublayer, squash, junction)
+        for i, L in enumerate(self.layers):
+            subs.append((i, 0, L.sq1, L.hc1))
+            if L.spec.mlp is not None:
+                subs.append((i, 1, L.sq2, L.hc2))
+        src, y, before = x0, None, None  # before: the sublayer whose output y has not been written to the streams yet
+        for i, sub, sq, hc in subs + [(len(self.layers), 0, self.final_squash, None)]:
+            h = torch.empty((T, W), dtype=self.dtype, device=dev)
+            last = hc is None
+            close = {} if before is None else dict(y=y, mix=before.mix, out_w=before.out, x_out=None if last and layer_outputs is None else xs)
+            mixops.stream_norm(src, n, read=None if last else hc.read, norm=sq.parts, scale=cfg.logit_scale if last else 1.0, h_out=h, **close)
+            if before is not None:
+                src = xs
+                if layer_outputs is not None and sub == 0:
+                    layer_outputs.append(xs.sum(dim=1))
+            if last:
+                return h
+            L = self.layers[i]
+            if sub == 1:
+                y = mixops.linear(mixops.clamp_gate(mixops.linear(h, L.up), L.spec.mlp.limit, L.spec.mlp.slope), L.down)
+            elif L.spec.kind == "diff_attention":
+                y = self._diff_attention(i, L, h, ctx, batch)
+            elif L.spec.kind in ("retention", "gla"):
+                y = self._decay_attention(i, L, h, ctx, batch)
+            else:
+                raise NotImplementedError(f"mixer {L.spec.kind!r} in a multi-stream stack")
+            before = hc
+        
 
     def _lightning(self, i: int, L: _Layer, h: torch.Tensor, ctx: Any, batch: Any) -> torch.Tensor:
         s, md = L.spec, batch.attn_metadata
@@ -1174,9 +1448,10 @@ class HybridDecoder:
         last token (prefill) or at every token (decode)."""
         cfg = self.cfg
         eps, alpha = cfg.rms_norm_eps, cfg.postln_alpha
-        if self.pre_norm or self.parallel or self.conv_stream:
-            hf = self._forward_pre_norm(ctx, batch, layer_outputs) if self.pre_norm else \
-                self._forward_parallel(ctx, batch, layer_outputs) if self.parallel else self._forward_conv(ctx, batch, layer_outputs)
+        if self.pre_norm or self.parallel or self.conv_stream or self.multi:
+            run = self._forward_pre_norm if self.pre_norm else self._forward_parallel if self.parallel else \
+                self._forward_conv if self.conv_stream else self._forward_streams
+            hf = run(ctx, batch, layer_outputs)
             rows = getattr(batch, "logit_rows", None)
             if rows is None and batch.is_prefill:
                 rows = batch.attn_metadata.get_last_indices(batch.size)

@@ -119,6 +119,10 @@ class HybridCache:
     * a model with a causal convolution of `taps` in front of every sublayer (`conv_in` = (taps, width)) keeps, per layer, sublayer and
       request, the last `taps - 1` normed rows in fp32: `conv_in_state(layer, sub)` is `[state_rows, taps - 1, width]` (all of them:
       `conv_in_states`, `[layers, 2, state_rows, taps - 1, width]`).
+    * a differential attention layer (`diff_attention`) caches keys and values like `attention`; a key head's row holds its two maps
+      side by side, so keys are `[slots, kv_heads * 2 * dim]` (every token stays cached, window and kept first tokens are applied when
+      reading);
+    * linear attention with decays (`retention`, `gla`) keeps the fp32 state `[state_rows, heads, dim, vdim]` like a lightning layer.
     Layers may differ in every size, so each gets its own allocation.  Every per-request row is indexed by the request's
     page-table row and needs no clearing: a request whose first token is at position 0 never reads what the row held.
     """
@@ -144,10 +148,10 @@ class HybridCache:
                 if spec.kv_from is None:
                     self._latent[i] = torch.zeros((slots, spec.kv_rank + spec.rot_dim), dtype=dtype, device=device)
                 self._owner[i] = i if spec.kv_from is None else spec.kv_from
-            elif spec.kind == "lightning":
+            elif spec.kind in ("lightning", "retention", "gla"):
                 self._state[i] = torch.zeros((state_rows, spec.heads, spec.dim, spec.vdim), dtype=torch.float32, device=device)
-            elif spec.kind in ("attention", "sink_attention"):
-                self._kv[i] = (torch.zeros((slots, spec.kv_heads * spec.dim), dtype=dtype, device=device),
+            elif spec.kind in ("attention", "sink_attention", "diff_attention"):
+                self._kv[i] = (torch.zeros((slots, spec.kv_heads * spec.maps * spec.dim), dtype=dtype, device=device),
                                torch.zeros((slots, spec.kv_heads * spec.vdim), dtype=dtype, device=device))
             elif spec.kind == "mamba1":
                 self._state[i] = torch.zeros((state_rows, spec.vdim, spec.dim), dtype=torch.float32, device=device)
@@ -194,7 +198,7 @@ class HybridCache:
     def bytes_per_page(layers, page_size: int, dtype: torch.dtype) -> int:
         es = torch.empty((), dtype=dtype).element_size()
         per_token = sum(s.kv_rank + s.rot_dim for s in layers if s.kind == "latent_attention" and s.kv_from is None)
-        per_token += sum(s.kv_heads * (s.dim + s.vdim) for s in layers if s.kind in ("attention", "sink_attention"))
+        per_token += sum(s.kv_heads * (s.maps * s.dim + s.vdim) for s in layers if s.kind in ("attention", "sink_attention", "diff_attention"))
         per_token += sum(s.left.kv_heads * (s.left.dim + s.left.vdim) for s in layers if s.kind == "parallel")
         return per_token * es * page_size
 
@@ -202,7 +206,8 @@ class HybridCache:
     def state_bytes(layers, state_rows: int, dtype: torch.dtype = torch.bfloat16, shift_width: int = 0, conv_in=(0, 0)) -> int:
         es = torch.empty((), dtype=dtype).element_size()
         taps_in, width_in = conv_in
-        total = sum(4 * s.heads * s.dim * s.vdim * state_rows for s in layers if s.kind in ("lightning", "delta", "channel_delta"))
+        total = sum(4 * s.heads * s.dim * s.vdim * state_rows for s in layers
+                    if s.kind in ("lightning", "delta", "channel_delta", "retention", "gla"))
         total += sum(es * (s.conv - 1) * (2 * s.kv_heads * s.dim + s.heads * s.vdim) * state_rows
                      for s in layers if s.kind in ("delta", "channel_delta"))
         for s in (x.right for x in layers if x.kind == "parallel"):

@@ -1,4 +1,4 @@
-"""torch-facing wrappers of the sequence-mixing kernels (include/msgl_mix.h, csrc/seqmix.hip, csrc/mix_delta.hip).
+"""torch-facing wrappers of the sequence-mixing kernels (include/msgl_mix.h, csrc/seqmix.hip, csrc/mix_*.hip).
 
 Same rules as ops.py: device tensors only, no CPU fallback, pointers + sizes + the current stream go straight to
 the C ABI.  `linear` is the projection seam of the hybrid models: the library GEMM (bf16, or fp32 in the library's
@@ -432,14 +432,14 @@ def delta_rule(out: torch.Tensor, qkv: torch.Tensor, state: torch.Tensor, b_raw:
         _p(None if first is None else _i32(first)), _p(scratch), _stream()), "delta_rule")
 
 
-def head_gated_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: float, H: int, dv: int, gate_act: int) -> torch.Tensor:
-    """Per head: o / rms(o) * weight[dv] * act(gate) -> [rows, H * dv] in the gate's dtype."""
+def head_gated_norm(o: torch.Tensor, gate: torch.Tensor, weight: Optional[torch.Tensor], eps: float, H: int, dv: int, gate_act: int) -> torch.Tensor:
+    """Per head: o / rms(o) * weight[dv] (None: ones) * act(gate) -> [rows, H * dv] in the gate's dtype."""
     _dev(o, gate, weight)
     rows = o.shape[0]
     assert o.dtype == torch.float32 and o.is_contiguous() and o.shape == (rows, H * dv) and gate.shape == (rows, H * dv)
-    assert gate.stride(1) == 1 and weight.dtype == gate.dtype and weight.shape == (dv,) and weight.is_contiguous()
+    assert gate.stride(1) == 1 and (weight is None or (weight.dtype == gate.dtype and weight.shape == (dv,) and weight.is_contiguous()))
     out = torch.empty((rows, H * dv), dtype=gate.dtype, device=o.device)
-    check_mix(mix_lib().msgl_mix_head_gated_norm(out.data_ptr(), o.data_ptr(), gate.data_ptr(), gate.stride(0), weight.data_ptr(),
+    check_mix(mix_lib().msgl_mix_head_gated_norm(out.data_ptr(), o.data_ptr(), gate.data_ptr(), gate.stride(0), _p(weight),
                                                  float(eps), rows, H, dv, gate_act, _code(gate), _stream()), "head_gated_norm")
     return out
 
@@ -514,15 +514,21 @@ def commit_rows(dst: Optional[torch.Tensor], src: Optional[torch.Tensor], slots:
 
 def qk_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor, out_loc: torch.Tensor,
             positions: torch.Tensor, cos_sin: Optional[torch.Tensor], eps: float, H: int, G: int, d: int, dv: int, *, interleaved: bool,
-            unit: bool, unit_v: bool = False) -> torch.Tensor:
+            unit: bool, unit_v: bool = False, norm_w=None, value_heads: Optional[int] = None) -> torch.Tensor:
     """Projection rows [q | k | v | ...] (+ fp32 bias) -> rotated (and unit-RMS) q as fp32 [T, H * d]; k, v into the cache rows
-    (unit_v: every value head divided by its root mean square first)."""
+    (unit_v: every value head divided by its root mean square first).  norm_w = (q weight, k weight), [d] each: q and k heads are
+    RMS-normed and multiplied by it before the rotation.  value_heads: how many value heads (default: as many as key heads)."""
     _dev(proj, bias, k_cache, v_cache, out_loc, positions, cos_sin)
     T = proj.shape[0]
-    n = (H + G) * d + G * dv
+    Gv = G if value_heads is None else value_heads
+    n = (H + G) * d + Gv * dv
     assert proj.stride(1) == 1 and proj.shape[1] >= n and (bias is None or _f32(bias, n) is not None)
-    assert k_cache.is_contiguous() and k_cache.shape[1] == G * d and v_cache.is_contiguous() and v_cache.shape[1] == G * dv
+    assert k_cache.is_contiguous() and k_cache.shape[1] == G * d and v_cache.is_contiguous() and v_cache.shape[1] == Gv * dv
     assert k_cache.dtype == proj.dtype == v_cache.dtype and out_loc.shape[0] == T
+    qw, kw = norm_w if norm_w is not None else (None, None)
+    for t in (qw, kw):
+        _dev(t)
+        assert t is None or (t.dtype == proj.dtype and t.is_contiguous() and t.shape == (d,))
     rd = 0
     if cos_sin is not None:
         assert cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.dim() == 2
@@ -530,7 +536,8 @@ def qk_prep(proj: torch.Tensor, bias: Optional[torch.Tensor], k_cache: torch.Ten
     q = torch.empty((T, H * d), dtype=torch.float32, device=proj.device)
     check_mix(mix_lib().msgl_mix_qk_prep(
         proj.data_ptr(), proj.stride(0), _p(bias), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), _i32(out_loc).data_ptr(),
-        _i32(positions).data_ptr(), _p(cos_sin), rd, int(interleaved), int(unit) | (2 if unit_v else 0), float(eps), T, H, G, d, dv, _code(proj), _stream()),
+        _i32(positions).data_ptr(), _p(cos_sin), rd, int(interleaved), int(unit) | (2 if unit_v else 0), float(eps),
+        _p(qw), _p(kw), T, H, G, Gv, d, dv, _code(proj), _stream()),
         "qk_prep")
     return q
 
@@ -681,7 +688,7 @@ def selective_scan(x: torch.Tensor, z: torch.Tensor, dt_in: torch.Tensor, bc: to
     return out
 
 
-def sink_attn_splits(batch: int, total_q: int, H: int, G: int, window: int, max_keys: int) -> int:
+def sink_attn_splits(batch: int, total_q: int, H: int, G: int, window: int, max_keys: int, keep: int = 0) -> int:
     """Key ranges per request for a step with few query rows: enough workgroups to fill the chip, at least 256 keys each.  A
     function of static sizes only (batch, rows, the window or the LONGEST possible key count), so a captured graph keeps its grid."""
     rep = H // G
@@ -689,15 +696,15 @@ def sink_attn_splits(batch: int, total_q: int, H: int, G: int, window: int, max_
     while hb * 2 <= min(rep, 64):
         hb *= 2
     blocks = (-(-total_q // (64 // hb)) + batch) * G * -(-rep // hb)
-    keys = min(window, max_keys) if window > 0 else max_keys
+    keys = min(window + keep, max_keys) if window > 0 else max_keys
     return max(1, min(1024 // max(blocks, 1), keys // 256, 64))
 
 
 def sink_attn(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, table: torch.Tensor, req_rows: torch.Tensor,
               seq_lens: torch.Tensor, cu_q: torch.Tensor, batch: int, H: int, G: int, d: int, dv: int, scale: float, window: int,
-              sink: Optional[torch.Tensor], splits: int = 1) -> None:
-    """out[:, : H * dv] = softmax attention over the last `window` keys (0: all earlier keys) with exp(sink[h]) as one more term of
-    the denominator (sink fp32 [H] or None)."""
+              sink: Optional[torch.Tensor], splits: int = 1, keep: int = 0) -> None:
+    """out[:, : H * dv] = softmax attention over the last `window` keys (0: all earlier keys) and the first `keep` ones, with
+    exp(sink[h]) as one more term of the denominator (sink fp32 [H] or None)."""
     _dev(out, q, k_cache, v_cache, table, req_rows, seq_lens, cu_q, sink)
     T = q.shape[0]
     assert q.dtype == torch.float32 and q.is_contiguous() and q.shape == (T, H * d)
@@ -711,7 +718,31 @@ def sink_attn(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache
     check_mix(mix_lib().msgl_mix_sink_attn(
         out.data_ptr(), out.stride(0), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), table.data_ptr(), table.stride(0),
         _i32(req_rows).data_ptr(), _i32(seq_lens).data_ptr(), _i32(cu_q).data_ptr(), batch, T, H, G, d, dv, float(scale), int(window),
-        _p(sink), _code(k_cache), splits, _p(ws), _stream()), "sink_attn")
+        int(keep), _p(sink), _code(k_cache), splits, _p(ws), _stream()), "sink_attn")
+
+
+def diff_attn(out: torch.Tensor, q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, table: torch.Tensor, req_rows: torch.Tensor,
+              seq_lens: torch.Tensor, cu_q: torch.Tensor, batch: int, H: int, G: int, d: int, dv: int, scale: float, window: int, keep: int,
+              lam: torch.Tensor, post: float, eps: float, gate: Optional[torch.Tensor] = None, splits: int = 1) -> None:
+    """Two softmax maps over the same values (q fp32 [T, H * 2 * d], key rows [G, 2, d], visible keys as in sink_attn): with their
+    outputs a1, a2 and lam (fp32 [1] on the device) out = rms_unit(a1 - lam a2) per head * post * sigmoid(gate) (gate [T, H * dv] in
+    out's dtype, a view with a row stride is fine, or None)."""
+    _dev(out, q, k_cache, v_cache, table, req_rows, seq_lens, cu_q, lam, gate)
+    T = q.shape[0]
+    assert q.dtype == torch.float32 and q.is_contiguous() and q.shape == (T, H * 2 * d)
+    assert out.shape == (T, H * dv) and out.stride(1) == 1 and out.dtype == k_cache.dtype == v_cache.dtype
+    assert k_cache.is_contiguous() and k_cache.shape[1] == G * 2 * d and v_cache.is_contiguous() and v_cache.shape[1] == G * dv
+    assert table.dtype == torch.int32 and table.stride(1) == 1 and _f32(lam, 1) is not None
+    assert gate is None or (gate.shape == (T, H * dv) and gate.stride(1) == 1 and gate.dtype == out.dtype)
+    assert req_rows.numel() >= batch and seq_lens.numel() >= batch and cu_q.numel() >= batch + 1
+    ws = None
+    if splits > 1:
+        ws = torch.empty(mix_lib().msgl_mix_sink_attn_workspace_floats(T, 2 * H, dv, splits), dtype=torch.float32, device=out.device)
+    check_mix(mix_lib().msgl_mix_diff_attn(
+        out.data_ptr(), out.stride(0), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), table.data_ptr(), table.stride(0),
+        _i32(req_rows).data_ptr(), _i32(seq_lens).data_ptr(), _i32(cu_q).data_ptr(), batch, T, H, G, d, dv, float(scale), int(window),
+        int(keep), lam.data_ptr(), float(post), float(eps), _p(gate), 0 if gate is None else gate.stride(0), _code(k_cache), splits, _p(ws),
+        _stream()), "diff_attn")
 
 
 def route_sigmoid(h: torch.Tensor, router: torch.Tensor, top: int):
@@ -773,3 +804,86 @@ def softcap(x: torch.Tensor, cap: float) -> torch.Tensor:
         return x
     check_mix(mix_lib().msgl_mix_softcap(x.data_ptr(), x.stride(0), x.shape[0], x.shape[1], float(cap), _code(x), _stream()), "softcap")
     return x
+
+
+# ------------------------------------------------------------------ multi-stream hybrid decoders (csrc/mix_streams.hip)
+def stream_norm(x: torch.Tensor, streams: int, *, y: Optional[torch.Tensor] = None, mix: Optional[torch.Tensor] = None,
+                out_w: Optional[torch.Tensor] = None, x_out: Optional[torch.Tensor] = None, read: Optional[torch.Tensor] = None,
+                norm=None, scale: float = 1.0, h_out: Optional[torch.Tensor] = None) -> None:
+    """x: fp32 [rows, streams, W], or [rows, W] standing for all streams.  With y [rows, W]: x'_t = sum_s mix[s, t] x_s + out_w[t] y ->
+    x_out (may be x itself when x has its streams).  h_out = (tanh(alpha u) w + b) * scale with u = sum_s read[s] x'_s (read None:
+    ones), norm = (w, b, alpha): w, b [W] in h_out's dtype, alpha fp32 [1]."""
+    bcast = x.dim() == 2
+    rows, W = x.shape[0], x.shape[-1]
+    _dev(x, y, mix, out_w, x_out, read, h_out)
+    assert x.dtype == torch.float32 and x.is_contiguous() and (bcast or x.shape == (rows, streams, W))
+    assert x_out is None or (x_out.dtype == torch.float32 and x_out.is_contiguous() and x_out.shape == (rows, streams, W))
+    _f32(out_w, streams), _f32(read, streams)
+    assert mix is None or (mix.dtype == torch.float32 and mix.is_contiguous() and mix.shape == (streams, streams))
+    w = b = alpha = None
+    dt = None
+    if h_out is not None:
+        w, b, alpha = norm
+        _dev(w, b, alpha)
+        dt = h_out.dtype
+        assert h_out.shape == (rows, W) and h_out.is_contiguous() and _f32(alpha, 1) is not None
+        for t in (w, b):
+            assert t.dtype == dt and t.is_contiguous() and t.shape == (W,)
+    if y is not None:
+        dt = dt or y.dtype
+        assert y.dtype == dt and y.is_contiguous() and y.shape == (rows, W) and mix is not None and out_w is not None
+    if rows:
+        check_mix(mix_lib().msgl_mix_stream_norm(
+            x.data_ptr(), int(bcast), _p(y), _p(mix), _p(out_w), _p(x_out), _p(read), _p(w), _p(b), _p(alpha), float(scale), _p(h_out), rows,
+            streams, W, _lib.BF16 if dt == torch.bfloat16 else _lib.F32, _stream()), "stream_norm")
+
+
+def decay_attn(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, state: torch.Tensor, cu_q: torch.Tensor,
+               seq_lens: torch.Tensor, slots: torch.Tensor, batch: int, eps: float, *, decay: Optional[torch.Tensor] = None,
+               z: Optional[torch.Tensor] = None, z_bias: Optional[torch.Tensor] = None, tau: float = 1.0, q_scale: float = 1.0,
+               k_scale: float = 1.0, cos_sin: Optional[torch.Tensor] = None, positions: Optional[torch.Tensor] = None,
+               interleaved: bool = False, weight: Optional[torch.Tensor] = None, chunks=None) -> torch.Tensor:
+    """S <- diag(a) S + k v^T, o = S^T q per (request, head); -> every head of o RMS-normed (times weight [dv]) and multiplied by
+    silu(gate), [T, H * dv] in the model dtype.  q, k [T, H * d], v, gate [T, H * dv]: column blocks of one projection; state fp32
+    [slots, H, d, dv].  Either decay (fp32 [H]) or z [T, H * d] with z_bias (fp32) and tau: a = sigmoid(z + z_bias)^(1 / tau) per key
+    channel.  cos_sin (fp32 [positions, rotated entries]): q and k turn first.  chunks = (items int32 [n, 3], item_first int32
+    [batch + 1], n) cuts long portions into pieces that run in parallel."""
+    _dev(q, k, v, gate, state, cu_q, seq_lens, slots, decay, z, z_bias, cos_sin, positions, weight)
+    _, H, d, dv = state.shape
+    T, dt = q.shape[0], q.dtype
+    assert state.dtype == torch.float32 and state.is_contiguous()
+    for t, n in ((q, H * d), (k, H * d), (v, H * dv), (gate, H * dv)):
+        assert t.shape == (T, n) and t.stride(1) == 1 and t.stride(0) == q.stride(0) and t.dtype == dt
+    assert (decay is None) != (z is None) and (decay is None or _f32(decay, H) is not None)
+    assert z is None or (z.shape == (T, H * d) and z.stride(1) == 1 and z.dtype == dt and _f32(z_bias, H * d) is not None and cos_sin is None)
+    assert weight is None or (weight.dtype == dt and weight.is_contiguous() and weight.shape == (dv,))
+    rd = 0
+    if cos_sin is not None:
+        assert cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.dim() == 2
+        rd = cos_sin.shape[1]
+    raw = not mix_lib().msgl_mix_decay_attn_fused(d, dv)
+    out = torch.empty((T, H * dv), dtype=torch.float32 if raw else dt, device=q.device)
+    items = first = scratch = None
+    n_items = 0
+    if chunks is not None:
+        items, first, n_items = chunks
+        _dev(items, first)
+        assert items.numel() == 3 * n_items and first.numel() == batch + 1
+        scratch = torch.empty(n_items * H * d * (dv + 1), dtype=torch.float32, device=q.device)
+    check_mix(mix_lib().msgl_mix_decay_attn(
+        out.data_ptr(), out.stride(0), int(raw), q.data_ptr(), k.data_ptr(), v.data_ptr(), gate.data_ptr(), q.stride(0), _p(z),
+        0 if z is None else z.stride(0), _p(z_bias), 1.0 / float(tau), _p(decay), float(q_scale), float(k_scale), _p(cos_sin),
+        _p(None if positions is None else _i32(positions)), rd, int(interleaved), _p(weight), float(eps), state.data_ptr(),
+        _i32(cu_q).data_ptr(), _i32(seq_lens).data_ptr(), _i32(slots).data_ptr(), batch, H, d, dv, _code(q), n_items,
+        _p(None if items is None else _i32(items)), _p(None if first is None else _i32(first)), _p(scratch), _stream()), "decay_attn")
+    return head_gated_norm(out, gate, weight, eps, H, dv, GATE_SILU) if raw else out
+
+
+def clamp_gate(gu: torch.Tensor, limit: float, slope: float) -> torch.Tensor:
+    """gu [rows, 2 N] = gate | up -> g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = clamp(up, -limit, limit)."""
+    _dev(gu)
+    rows, N = gu.shape[0], gu.shape[1] // 2
+    assert gu.is_contiguous() and gu.shape == (rows, 2 * N)
+    out = torch.empty((rows, N), dtype=gu.dtype, device=gu.device)
+    check_mix(mix_lib().msgl_mix_clamp_gate(out.data_ptr(), gu.data_ptr(), rows, N, float(limit), float(slope), _code(gu), _stream()), "clamp_gate")
+    return out

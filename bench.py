@@ -682,7 +682,17 @@ def main() -> None:
                          "hybrid decoder of equal size, and its kernels against their rooflines (tools/piladra_bench.py; further flags "
                          "after --piladra-args)")
     ap.add_argument("--piladra-args", nargs=argparse.REMAINDER, default=[], help="flags handed to tools/piladra_bench.py")
+    ap.add_argument("--nagezen", action="store_true",
+                    help="instead of the default workload: prefill / decode throughput of the multi-stream hybrid decoder (retention, gated "
+                         "linear attention, two-map windowed attention) beside the looped pre-norm hybrid decoder of equal size, and its "
+                         "kernels against their rooflines (tools/nagezen_bench.py; further flags after --nagezen-args)")
+    ap.add_argument("--nagezen-args", nargs=argparse.REMAINDER, default=[], help="flags handed to tools/nagezen_bench.py")
     args = ap.parse_args()
+    if args.nagezen:
+        from tools.nagezen_bench import main as nagezen_main
+
+        nagezen_main(list(args.nagezen_args))
+        return
     if args.bedarax:
         from tools.bedarax_bench import main as bedarax_main
 

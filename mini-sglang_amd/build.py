@@ -101,42 +101,25 @@ def build_all(force: bool = False, verbose: bool = True, only=None) -> dict[str,
     LIB.mkdir(exist_ok=True)
     OBJ.mkdir(exist_ok=True)
 
-    def srcs(key, names):
-        return [CSRC / s for s in names if (CSRC / s).exists()] if key in want else []
-
-    hip_srcs, mix_srcs = srcs("hip", HIP_SOURCES), srcs("mix", MIX_SOURCES)
-    comm_srcs, gemm_srcs = srcs("comm", COMM_SOURCES), srcs("gemm", GEMM_SOURCES)
-    groups = [hip_srcs, mix_srcs, comm_srcs, gemm_srcs]
-    with ThreadPoolExecutor(max_workers=min(8, os.cpu_count() or 1)) as pool:
-        objs = list(pool.map(lambda s: _compile(s, force), [s for g in groups for s in g]))
-    cut = [0]
-    for g in groups:
-        cut.append(cut[-1] + len(g))
-    hip_objs, mix_objs, comm_objs, gemm_objs = (objs[cut[i]: cut[i + 1]] for i in range(4))
-    out = {}
-    # --no-undefined: a kernel whose host-side launch stub went missing must fail HERE, not at dlopen on the GPU box
-    if hip_objs:
-        lib_hip = LIB / "libmsgl_hip.so"
-        if force or _stale(lib_hip, hip_objs):
-            _run([HIPCC, "-shared", "-fPIC", f"--offload-arch={ARCH}", "-Wl,--no-undefined", *map(str, hip_objs), "-o", str(lib_hip)])
-        out["hip"] = lib_hip
-    if mix_objs:
-        lib_mix = LIB / "libmsgl_mix.so"
-        if force or _stale(lib_mix, mix_objs):
-            _run([HIPCC, "-shared", "-fPIC", f"--offload-arch={ARCH}", "-Wl,--no-undefined", *map(str, mix_objs), "-o", str(lib_mix)])
-        out["mix"] = lib_mix
-    if comm_objs:
-        lib_comm = LIB / "libmsgl_comm.so"
-        if force or _stale(lib_comm, comm_objs):
-            _run([HIPCC, "-shared", "-fPIC", *map(str, comm_objs), "-L", str(ROCM / "lib"), "-lrccl",
-                  f"-Wl,-rpath,{ROCM / 'lib'}", "-o", str(lib_comm)])
-        out["comm"] = lib_comm
-    if gemm_objs:
-        lib_gemm = LIB / "libmsgl_gemm.so"
-        if force or _stale(lib_gemm, gemm_objs):
-            _run([HIPCC, "-shared", "-fPIC", *map(str, gemm_objs), "-L", str(ROCM / "lib"), "-lhipblaslt",
-                  f"-Wl,-rpath,{ROCM / 'lib'}", "-o", str(lib_gemm)])
-        out["gemm"] = lib_gemm
+    # library -> (its sources, its link line); a library newer than its sources and the headers is left alone, object files or not
+    # (a checkout that ships built libraries does not ship the objects)
+    link = [HIPCC, "-shared", "-fPIC"]
+    libs = {
+        # --no-undefined: a kernel whose host-side launch stub went missing must fail HERE, not at dlopen on the GPU box
+        "hip": (HIP_SOURCES, [*link, f"--offload-arch={ARCH}", "-Wl,--no-undefined"], []),
+        "mix": (MIX_SOURCES, [*link, f"--offload-arch={ARCH}", "-Wl,--no-undefined"], []),
+        "comm": (COMM_SOURCES, link, ["-L", str(ROCM / "lib"), "-lrccl", f"-Wl,-rpath,{ROCM / 'lib'}"]),
+        "gemm": (GEMM_SOURCES, link, ["-L", str(ROCM / "lib"), "-lhipblaslt", f"-Wl,-rpath,{ROCM / 'lib'}"]),
+    }
+    headers = list(CSRC.glob("*.h")) + list(INCLUDE.glob("*.h"))
+    out = {k: LIB / f"libmsgl_{k}.so" for k in libs if k in want}
+    todo = {k: [CSRC / n for n in libs[k][0]] for k in out}
+    todo = {k: srcs for k, srcs in todo.items() if force or _stale(out[k], srcs + headers)}
+    with ThreadPoolExecutor(max_workers=min(16, os.cpu_count() or 1)) as pool:
+        objs = {k: [pool.submit(_compile, s, force) for s in srcs] for k, srcs in todo.items()}
+        for k, futures in objs.items():
+            built = [str(f.result()) for f in futures]
+            _run([*libs[k][1], *built, *libs[k][2], "-o", str(out[k])])
     if verbose:
         for k, v in out.items():
             print(f"[build] {k}: {v} ({v.stat().st_size >> 10} KiB)")

@@ -608,7 +608,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
 constexpr int kNKT = 64;
 
 template <int KC, int VC, int MAPS>
-__global__ __launch_bounds__(256) void sink_attn_mfma_kernel(bf16_t* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
+__global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void sink_attn_mfma_kernel(bf16_t* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
                                                              float* __restrict__ part_ml, const float* __restrict__ q,
                                                              const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
                                                              const int* __restrict__ table, int64_t table_stride,

@@ -172,7 +172,7 @@ struct DecayArgs {
 };
 
 template <typename T, bool CHANNEL, int DT, int NS>
-__global__ __launch_bounds__(256) void decay_attn_kernel(DecayArgs a) {
+__global__ __launch_bounds__(256, DT * NS <= 16 ? 2 : 1) void decay_attn_kernel(DecayArgs a) {
   constexpr int DP = DT * 16, LD = DP + 4;
   // staging: HEAD: a thread takes one (rotation) pair of entries of TP tokens; CHANNEL: one channel of TP tokens
   constexpr int kCols = CHANNEL ? DP : DP / 2, kParts = 256 / kCols, TP = kPiece / kParts;

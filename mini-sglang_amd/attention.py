@@ -227,7 +227,6 @@ class MixAttnBackend:
     DELTA_CHUNK = 256
     SSD_CHUNK = 64
     SCAN_CHUNK = 64
-    DECAY_CHUNK = 128
 
     def __init__(self, config: Any, ctx: Any = None, *, tp_size: int = 1) -> None:
         ctx = ctx if ctx is not None else _core.get_global_ctx()
@@ -238,7 +237,14 @@ class MixAttnBackend:
         self.capture_bs: List[int] = []
         self._cap: Optional[torch.Tensor] = None
         self._kinds = {getattr(s, "kind", "") for s in getattr(config, "layers", ())}
+        self._decay_heads = max((s.heads for s in getattr(config, "layers", ()) if getattr(s, "kind", "") in ("retention", "gla")), default=0)
         self._kinds |= {getattr(p, "kind", "") for s in getattr(config, "layers", ()) for p in (getattr(s, "left", None), getattr(s, "right", None)) if p}
+
+    @staticmethod
+    def decay_chunk(tokens: int, heads: int) -> int:
+        """Piece size of the decay recurrences in a step of `tokens` new tokens: as many (piece, head) workgroups as the chip holds at a
+        time (two per compute unit), in whole 16-token pieces, between 32 and 512 tokens."""
+        return min(max(-(-tokens * heads // (512 * 16)) * 16, 32), 512)
 
     def prepare_metadata(self, batch: Any) -> None:
         reqs = batch.padded_reqs
@@ -257,8 +263,10 @@ class MixAttnBackend:
             lists.append(("ssd_chunks", self.SSD_CHUNK))
         if int(q.max()) >= 2 * self.SCAN_CHUNK and "mamba1" in self._kinds:
             lists.append(("scan_chunks", self.SCAN_CHUNK))
-        if int(q.max()) >= 2 * self.DECAY_CHUNK and self._kinds & {"retention", "gla"}:
-            lists.append(("decay_chunks", self.DECAY_CHUNK))
+        if self._decay_heads:
+            c = self.decay_chunk(int(q.sum()), self._decay_heads)
+            if int(q.max()) >= 2 * c:
+                lists.append(("decay_chunks", c))
         pieces = [-(-q // c) for _, c in lists]
         extra = sum(3 * int(p.sum()) + bs + 1 for p in pieces)
         host = torch.empty(3 * bs + 1 + extra, dtype=torch.int32, pin_memory=True)

@@ -130,7 +130,7 @@ def kernel_rooflines(name: str, prompt: int, batch: int, device, chunk: int = 0)
         tab = torch.rand(ctx, D, device=device)
         byts = 2 * reqs * H * D * D * 4 + T * H * D * 2 * 5
         flops = 4.0 * T * H * D * D  # the update and the read of the state; what a piece does besides is the kernel's own choice
-        ch = chunk_list(q_len, reqs, chunk or MixAttnBackend.DECAY_CHUNK)
+        ch = chunk_list(q_len, reqs, chunk or MixAttnBackend.decay_chunk(T, H))
         us = _time_us(lambda: mixops.decay_attn(*cols, state, cu, seq, rows, reqs, 1e-5, decay=decay, k_scale=D ** -0.5, cos_sin=tab, positions=pos, chunks=ch))
         out[f"{phase}.decay_attn (per head)"] = _entry(us, flops, byts, VALU_TFLOPS)
         z, zb, w = rnd(T, H * D), torch.ones(H * D, device=device), rnd(D)

@@ -81,16 +81,16 @@ def _run(cmd: list[str]) -> None:
         sys.stderr.write(proc.stderr)
 
 
-# fp32 arithmetic stays scalar in the sequence-mixing kernels: no packed two-lane fp32 instructions (a device-pass flag;
-# the host pass says it does not know the feature, which is harmless)
-MIX_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+# fp32 arithmetic stays scalar: no packed two-lane fp32 instructions in any kernel (a device-pass flag; the host pass says it does
+# not know the feature, which is harmless)
+KERNEL_FLAGS = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 
 def _compile(src: Path, force: bool) -> Path:
     obj = OBJ / (src.name + ".o")
     headers = list(CSRC.glob("*.h")) + list(INCLUDE.glob("*.h"))
     if force or _stale(obj, [src] + headers):
-        extra = MIX_FLAGS if src.name in MIX_SOURCES else []
+        extra = KERNEL_FLAGS if src.suffix == ".hip" else []
         _run([HIPCC, *COMMON_FLAGS, *extra, "-x", "hip", "-c", str(src), "-o", str(obj)])
     return obj
 

@@ -19,7 +19,7 @@
 //     reduce-scatter over a role-ordered tile (see the kernel): 5 G DPP adds per tile instead
 //     of 16 G, the softmax scalar work (scale, max, exp) is done once per token instead of
 //     once per lane, probabilities of the row's other three tokens return by 3 G DPP moves,
-//     P.V with v_pk_fma_f32; softmax state (m, o) per 16-lane row over its token subset, l per
+//     P.V with fp32 FMA; softmax state (m, o) per 16-lane row over its token subset, l per
 //     quad, merged once per unit.  (The all-reduce formulation it replaces measured the same
 //     at G = 5 and 20 % slower at G = 8: profiles/r01c_microbench_decode_rs{0,1}.json.)
 //   * K/V tiles double-buffered in registers one 16-token tile ahead (8 KB in flight per

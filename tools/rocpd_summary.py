@@ -12,7 +12,7 @@ import sys
 
 
 def short(name: str) -> str:
-    name = re.sub(r"\[clone .*\]", "", name)
+    name = re.sub(r"\[clone .*\]", "", name).replace("(anonymous namespace)::", "")
     name = re.sub(r"\(.*", "", name)
     return name.strip()[:110]
 

@@ -111,6 +111,16 @@ def test_checkpoint_round_trip_and_cache_layout():
     assert HybridCache.state_bytes(layers, 3, torch.bfloat16) == 4 * 3 * (2 * 5 * 9 + 3 * 6 * 10)
 
 
+def test_piece_size_of_the_recurrences():
+    from mini_sglang_amd.attention import MixAttnBackend
+
+    for tokens, heads in ((1, 1), (300, 3), (2048, 8), (8192, 16), (65536, 64)):
+        c = MixAttnBackend.decay_chunk(tokens, heads)
+        assert c % 16 == 0 and 32 <= c <= 512
+        assert c == 512 or -(-tokens // c) * heads <= 512 or c == 32
+    assert MixAttnBackend.decay_chunk(2048, 16) == 64
+
+
 def test_restatement_by_hand():
     f = torch.float64
     # two streams, (1, 10) and (2, 20): read (0.5, 2); mixing rows are where a stream comes FROM

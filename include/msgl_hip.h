@@ -45,6 +45,7 @@ extern "C" {
 #define MSGL_FP16 1
 /* dtype codes for logits */
 #define MSGL_F32 2
+#define MSGL_BF16_OUT_F32 3 /* msgl_gemm_nt only: bf16 operands, fp32 result */
 
 #define MSGL_ABI_VERSION 5
 

@@ -1,7 +1,7 @@
 /*
  * msgl_mix.h -- C ABI of the sequence-mixing kernels (latent attention, linear-recurrence layers, routed experts)
  * for gfx950; implemented by libmsgl_mix.so (mini-sglang_amd/csrc/seqmix.hip, mix_delta.hip, mix_par.hip,
- * mix_scan.hip, mix_streams.hip).
+ * mix_scan.hip, mix_streams.hip, mix_sandwich.hip).
  *
  * Same conventions as msgl_hip.h: raw device pointers, explicit sizes and strides in ELEMENTS, `stream` is a
  * hipStream_t passed as void*, every function returns 0 or a negative code and leaves a message for
@@ -28,7 +28,10 @@ extern "C" {
 #define MSGL_MIX_ACT_NONE 0
 #define MSGL_MIX_ACT_RELU2 1 /* max(z, 0)^2 */
 
-#define MSGL_MIX_ABI_VERSION 5
+#define MSGL_MIX_GATE_MUL_SILU 0
+#define MSGL_MIX_GATE_MUL_GELU_TANH 1
+
+#define MSGL_MIX_ABI_VERSION 6
 
 const char* msgl_mix_last_error(void);
 int msgl_mix_abi_version(void);
@@ -83,10 +86,11 @@ int msgl_mix_gated_norm(void* out, const float* o, const void* gate, int64_t ld_
                         void* stream);
 
 /* Router on fp32 logits z [tokens, E] (= router weights x the token, accumulated in fp32 by a product kernel): s = softmax(z);
- * choice = s + bias (bias in T, may be null); only experts of the `keep` best of G equal groups of neighbours (group score = its
- * largest choice) can win; ids = the `top` largest choices, wts = their s / (sum + 1e-20). */
-int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int tokens, int E, int top, int G, int keep, int dtype,
-                   void* stream);
+ * choice = s + bias (bias in T, may be null); only experts of the `keep` best of G equal groups of neighbours (group score = the
+ * sum of its `group_best` largest choices, 1 or 2) can win; ids = the `top` largest choices, wts = their s / (sum + 1e-20) * scale.
+ * sigmoid != 0: s = sigmoid(z) expert by expert in the place of the softmax. */
+int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int tokens, int E, int top, int G, int keep, int sigmoid,
+                   int group_best, float scale, int dtype, void* stream);
 
 /* seg[E + 1], perm[n]: flat (token, choice) indices bucketed by expert, stable inside a bucket; counts[E] is scratch. */
 int msgl_mix_moe_sort(int* seg, int* perm, int* counts, const int* ids, int n, int E, void* stream);
@@ -116,9 +120,6 @@ int msgl_mix_prenorm(const float* x_in, const void* y, int parts, const float* g
 /* out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 over rows of N (powers element-wise, N(.) = the row divided by its root mean
  * square, eps inside the root); coef: 4 floats on the device. */
 int msgl_mix_poly_act(void* out, const void* z, int64_t ldz, const float* coef, float eps, int rows, int N, int dtype, void* stream);
-
-/* out[r, i] = silu(gate_up[r, i]) * gate_up[r, N + i]  (rows of 2 N -> rows of N). */
-int msgl_mix_silu_mul(void* out, const void* gate_up, int rows, int N, int dtype, void* stream);
 
 /* Router on fp32 logits z [tokens, E] (+ bias in T, may be null): ids = the `top` largest logits (ties: lowest index, in
  * descending order), wts = softmax over those logits only. */
@@ -316,6 +317,23 @@ int msgl_mix_decay_attn(void* out, int64_t ld_out, int raw, const void* q, const
 
 /* gu: T rows [gate: N | up: N];  out (T [rows, N]) = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = clamp(up, -limit, limit). */
 int msgl_mix_clamp_gate(void* out, const void* gu, int rows, int N, float limit, float slope, int dtype, void* stream);
+
+/* ---- decoders that norm a sublayer's input and its output (csrc/mix_sandwich.hip) ---- */
+
+/* Closes a sublayer and opens the next.  N(v) = (v - mean(v)) / sqrt(mean((v - mean(v))^2) + eps), with centre = 0 the mean counts as 0.
+ *   x  = x_in[t] (fp32 [rows, W]), or scale * table[ids[t]] (T) when x_in is null;
+ *   s  = sum_p gate[t, p] y0[t, p] (T [rows, p0, W]; gate fp32 [rows, p0], null: ones) + y1[t] (T [rows, W]); each may be absent;
+ *   x' = x + N(s) * w_in (w_in T [W]; null: x + s)  -> x_out (fp32, may be x_in) and, as T rows ld_raw apart, raw0 and raw1 (all optional);
+ *   h  = N(x') * w_out -> h_out (T [rows, W]; both null: none).
+ * router != null (T [E, W]; h_out required): h (its copy in T) is routed in the same launch, logits in fp32, choice and weights as in
+ * msgl_mix_route (bias T [E] or null, route_scale = its scale) -> pick int32 [rows, top], wts fp32 [rows, top]. */
+int msgl_mix_join_norm(const float* x_in, const void* table, const int* ids, float scale, const void* y0, int p0, const float* gate,
+                       const void* y1, const void* w_in, float* x_out, void* raw0, void* raw1, int64_t ld_raw, const void* w_out, void* h_out,
+                       float eps, int centre, int rows, int W, int dtype, const void* router, const void* bias, int E, int top, int G, int keep,
+                       int sigmoid, int group_best, float route_scale, int* pick, float* wts, void* stream);
+
+/* gu: T rows [gate: N | up: N];  out (T [rows, N]) = act(gate) * up. */
+int msgl_mix_gate_mul(void* out, const void* gu, int rows, int N, int act, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

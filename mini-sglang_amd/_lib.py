@@ -20,9 +20,9 @@ HIP_SO = LIB_DIR / "libmsgl_hip.so"
 COMM_SO = LIB_DIR / "libmsgl_comm.so"
 GEMM_SO = LIB_DIR / "libmsgl_gemm.so"
 MIX_SO = LIB_DIR / "libmsgl_mix.so"
-MIX_ABI_VERSION = 5
+MIX_ABI_VERSION = 6
 
-BF16, FP16, F32 = 0, 1, 2
+BF16, FP16, F32, BF16_OUT_F32 = 0, 1, 2, 3
 UNIQUE_ID_BYTES = 128
 IPC_HANDLE_BYTES = 64
 PREFILL_QTILE = 128
@@ -150,13 +150,12 @@ MIX_SIGNATURES = {
     "msgl_mix_latent_attn": (_i, [_p, _p, _p, _p, _l, _p, _p, _p, _i, _i, _i, _i, _i, _f, _p, _i, _i, _p, _p]),
     "msgl_mix_lightning": (_i, [_p, _p, _l, _p, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _p, _p, _p, _p]),
     "msgl_mix_gated_norm": (_i, [_p, _p, _p, _l, _p, _f, _i, _i, _i, _p]),
-    "msgl_mix_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _p]),
+    "msgl_mix_route": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _i, _i, _i, _f, _i, _p]),
     "msgl_mix_moe_sort": (_i, [_p, _p, _p, _p, _i, _i, _p]),
     "msgl_mix_gemm_nt": (_i, [_p, _p, _p, _i, _i, _i, _l, _l, _l, _i, _l, _l, _l, _p, _p, _i, _p, _i, _i, _i, _i, _p]),
     "msgl_mix_embed_norm": (_i, [_p, _p, _p, _p, _f, _i, _i, _i, _p]),
     "msgl_mix_prenorm": (_i, [_p, _p, _i, _p, _p, _p, _l, _p, _i, _p, _p, _p, _f, _i, _i, _i, _p, _p, _i, _i, _p, _p, _p]),
     "msgl_mix_poly_act": (_i, [_p, _p, _l, _p, _f, _i, _i, _i, _p]),
-    "msgl_mix_silu_mul": (_i, [_p, _p, _i, _i, _i, _p]),
     "msgl_mix_route_top": (_i, [_p, _p, _p, _p, _i, _i, _i, _i, _p]),
     "msgl_mix_kv_store": (_i, [_p, _p, _p, _p, _l, _i, _i, _i, _i, _p, _l, _p, _i, _i, _p]),
     "msgl_mix_window_attn_workspace_floats": (_i, [_i, _i, _i, _i]),
@@ -188,6 +187,8 @@ MIX_SIGNATURES = {
     "msgl_mix_decay_attn": (_i, [_p, _l, _i, _p, _p, _p, _p, _l, _p, _l, _p, _f, _p, _f, _f, _p, _p, _i, _i, _p, _f, _p, _p, _p, _p, _i, _i, _i, _i, _i, _i,
                                  _p, _p, _p, _p]),
     "msgl_mix_clamp_gate": (_i, [_p, _p, _i, _i, _f, _f, _i, _p]),
+    "msgl_mix_join_norm": (_i, [_p, _p, _p, _f, _p, _i, _p, _p, _p, _p, _p, _p, _l, _p, _p, _f, _i, _i, _i, _i, _p, _p, _i, _i, _i, _i, _i, _i, _f, _p, _p, _p]),
+    "msgl_mix_gate_mul": (_i, [_p, _p, _i, _i, _i, _i, _p]),
 }
 
 

@@ -155,7 +155,8 @@ int get_handle(hipblasLtHandle_t* h, int* dev_out) {
 
 int make_problem(Problem* p, int M, int N, int K, int64_t ldx, int64_t ldw, int64_t ldo, int dtype) {
   // fp32 operands run with HIPBLAS_COMPUTE_32F, the library's true 32-bit mode (no reduced-precision matrix format)
-  const hipDataType t = dtype == MSGL_F32 ? HIP_R_32F : dtype == MSGL_BF16 ? HIP_R_16BF : HIP_R_16F;
+  const hipDataType t = dtype == MSGL_F32 ? HIP_R_32F : dtype == MSGL_FP16 ? HIP_R_16F : HIP_R_16BF;
+  const hipDataType td = dtype == MSGL_BF16_OUT_F32 ? HIP_R_32F : t;
   GEMM_BLAS(hipblasLtMatmulDescCreate(&p->desc, HIPBLAS_COMPUTE_32F, HIP_R_32F));
   const int32_t ta = HIPBLAS_OP_T, tb = HIPBLAS_OP_N;
   GEMM_BLAS(hipblasLtMatmulDescSetAttribute(p->desc, HIPBLASLT_MATMUL_DESC_TRANSA, &ta, sizeof(ta)));
@@ -165,7 +166,7 @@ int make_problem(Problem* p, int M, int N, int K, int64_t ldx, int64_t ldw, int6
   // B = X stored [M][K] row-major = column-major K x M with ld = ldx
   GEMM_BLAS(hipblasLtMatrixLayoutCreate(&p->b, t, (uint64_t)K, (uint64_t)M, ldx));
   // D = out stored [M][N] row-major = column-major N x M with ld = ldo
-  GEMM_BLAS(hipblasLtMatrixLayoutCreate(&p->d, t, (uint64_t)N, (uint64_t)M, ldo));
+  GEMM_BLAS(hipblasLtMatrixLayoutCreate(&p->d, td, (uint64_t)N, (uint64_t)M, ldo));
   return MSGL_OK;
 }
 
@@ -175,7 +176,7 @@ int check_args(const void* out, const void* x, const void* w, int M, int N, int 
   GEMM_REQUIRE(M >= 1 && N >= 1 && K >= 1, "gemm: bad shape %d x %d x %d", M, N, K);
   GEMM_REQUIRE(ldx >= K && ldw >= K && ldo >= N, "gemm: leading dimensions (%lld, %lld, %lld) too small",
                (long long)ldx, (long long)ldw, (long long)ldo);
-  GEMM_REQUIRE(dtype == MSGL_BF16 || dtype == MSGL_FP16 || dtype == MSGL_F32, "gemm: unsupported dtype code %d", dtype);
+  GEMM_REQUIRE(dtype == MSGL_BF16 || dtype == MSGL_FP16 || dtype == MSGL_F32 || dtype == MSGL_BF16_OUT_F32, "gemm: unsupported dtype code %d", dtype);
   return MSGL_OK;
 }
 
@@ -259,6 +260,7 @@ int msgl_gemm_tune(void* out, const void* x, const void* const* w_list, int n_w,
   GEMM_REQUIRE(w_list && n_w >= 1, "gemm_tune: need at least one weight buffer");
   int rc = check_args(out, x, w_list[0], M, N, K, ldx, ldw, ldo, dtype);
   if (rc != MSGL_OK) return rc;
+  GEMM_REQUIRE(dtype != MSGL_BF16_OUT_F32, "gemm_tune: operands and result share one dtype");
   if (iters < 1) iters = 1;
   std::lock_guard<std::mutex> lock(g_mu);
   hipblasLtHandle_t h;

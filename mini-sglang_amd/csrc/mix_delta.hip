@@ -11,7 +11,6 @@
 //   prenorm_kernel           s = x + sum_p g[t,p] y[t,p];  optional depth average over the stored history;  h = rms(.) * w;
 //                            ROUTE: logits of the normed row, top-`top` by logit, softmax over the chosen ones
 //   poly_act_kernel          a N(z) + b N(z^2) + c N(z^3) + e,  N = divide a row by its root mean square
-//   silu_mul_kernel          silu(gate) * up over rows [gate | up]
 //   route_top_kernel         stand-alone router on given fp32 logits (long batches)
 //   kv_store_kernel          k and the (blended) v of a token -> cache rows at out_loc
 //   window_attn_kernel       sliding-window attention over the paged rows: raw scores of all heads, mixed by the H x H table,
@@ -245,16 +244,6 @@ __global__ __launch_bounds__(256) void poly_act_kernel(T* __restrict__ out, cons
     const float v = ld(z + (size_t)t * ldz + i);
     st(out + (size_t)t * N + i, a * v + b * (v * v) + c * (v * v * v) + e);
   }
-}
-
-template <typename T>
-__global__ __launch_bounds__(256) void silu_mul_kernel(T* __restrict__ out, const T* __restrict__ gu, int64_t total, int N) {
-  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-  if (i >= total) return;
-  const int64_t r = i / N;
-  const int col = (int)(i - r * N);
-  const T* row = gu + r * 2 * N;
-  st(out + i, siluf_(ld(row + col)) * ld(row + N + col));
 }
 
 // ------------------------------------------------------------------------------------------------ cache rows of the windowed attention
@@ -849,17 +838,6 @@ int msgl_mix_poly_act(void* out, const void* z, int64_t ldz, const float* coef, 
   hipStream_t s = static_cast<hipStream_t>(stream);
   DISPATCH_T(dtype, hipLaunchKernelGGL(poly_act_kernel<T>, dim3(rows), dim3(256), 0, s, mp<T>(out), cp<T>(z), ldz, coef, eps, N);)
   MIX_LAUNCHED("poly_act");
-  return MSGL_MIX_OK;
-}
-
-int msgl_mix_silu_mul(void* out, const void* gate_up, int rows, int N, int dtype, void* stream) {
-  MIX_REQUIRE(out && gate_up && rows >= 0 && N >= 1 && dtype_ok(dtype), "silu_mul: bad arguments");
-  if (rows == 0) return MSGL_MIX_OK;
-  const int64_t total = (int64_t)rows * N;
-  hipStream_t s = static_cast<hipStream_t>(stream);
-  DISPATCH_T(dtype, hipLaunchKernelGGL(silu_mul_kernel<T>, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, s, mp<T>(out),
-                                       cp<T>(gate_up), total, N);)
-  MIX_LAUNCHED("silu_mul");
   return MSGL_MIX_OK;
 }
 

@@ -20,7 +20,7 @@
 //   gemm_nt_mfma_kernel      grouped / segmented / gathered C = act(A B^T) for 16-bit weights on the matrix cores: per-head
 //                            latent products, expert layers, router logits of long batches
 //   gemm_nt_kernel           the same in fp32 FMA: fp32 engines, and every shape the library refuses
-#include "mix_common.h"
+#include "mix_route.h"
 
 namespace {
 
@@ -365,141 +365,12 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ out, co
 
 // ------------------------------------------------------------------------------------------------ router
 // One thread per token over router logits z [T, E] that a product kernel wrote in fp32 (bf16 x bf16 products are exact in fp32,
-// so the matrix cores' fp32 accumulation IS the 32-bit router on the token's 16-bit copy).  s = softmax(z); choice = s + bias;
-// experts outside the `keep` best groups (a group's score = its largest choice) are out; the `top` largest choices win (ties:
-// lowest index); weight = s / (sum of chosen s + 1e-20).  Scores live in LDS columns, one per thread.
-// s[e * st] holds the router logits of one token on entry (st = column stride: one column per thread); c is scratch of the
-// same shape, gs of G entries.  Writes the token's `top` expert ids and weights.
-template <typename T>
-__device__ __forceinline__ void select_experts(float* s, float* c, float* gs, int st, const T* __restrict__ bias, int E, int top, int G,
-                                               int keep, int* __restrict__ ids, float* __restrict__ wts) {
-  float mx = -INFINITY;
-  for (int e = 0; e < E; ++e) mx = fmaxf(mx, s[e * st]);
-  float sum = 0.f;
-  for (int e = 0; e < E; ++e) {
-    const float v = expf(s[e * st] - mx);
-    s[e * st] = v;
-    sum += v;
-  }
-  for (int e = 0; e < E; ++e) {
-    const float v = s[e * st] / sum;
-    s[e * st] = v;
-    c[e * st] = v + (bias ? ld(bias + e) : 0.f);
-  }
-  const int per = E / G;
-  if (keep < G) {
-    // a group's score = its largest choice; it stays if fewer than `keep` groups beat it (ties: the lower index wins)
-    for (int g = 0; g < G; ++g) {
-      float best = -INFINITY;
-      for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, c[e * st]);
-      gs[g * st] = best;
-    }
-    for (int g = 0; g < G; ++g) {
-      const float mine = gs[g * st];
-      int better = 0;
-      for (int o2 = 0; o2 < G; ++o2) better += (gs[o2 * st] > mine) || (gs[o2 * st] == mine && o2 < g);
-      if (better >= keep)
-        for (int e = g * per; e < (g + 1) * per; ++e) c[e * st] = -INFINITY;
-    }
-  }
-  float tot = 0.f;
-  for (int k = 0; k < top; ++k) {
-    int best = -1;
-    float bv = -INFINITY;
-    for (int e = 0; e < E; ++e) {
-      const float v = c[e * st];
-      if (v > bv) {
-        best = e;
-        bv = v;
-      }
-    }
-    if (best < 0) best = 0;  // unreachable: the host checks top <= keep * (E / G) and choice scores are finite
-    ids[k] = best;
-    const float sv = s[best * st];
-    wts[k] = sv;
-    tot += sv;
-    c[best * st] = -INFINITY;
-  }
-  for (int k = 0; k < top; ++k) wts[k] /= (tot + 1e-20f);
-}
-
-// The same selection by the 64 lanes of one wave over one token (lane owns experts lane, lane + 64, ...): reductions by
-// lane exchange in a fixed order, so the result does not depend on anything but the logits.  s, c: E entries of LDS each, gs: G + top.
-__device__ __forceinline__ float wave_max_f(float v) {
-#pragma unroll
-  for (int o = 32; o >= 1; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
-  return v;
-}
-template <typename T>
-__device__ __forceinline__ void select_experts_wave(float* s, float* c, float* gs, const T* __restrict__ bias, int E, int top, int G,
-                                                    int keep, int* __restrict__ ids, float* __restrict__ wts) {
-  const int lane = threadIdx.x & 63;
-  float mx = -INFINITY;
-  for (int e = lane; e < E; e += 64) mx = fmaxf(mx, s[e]);
-  mx = wave_max_f(mx);
-  float sum = 0.f;
-  for (int e = lane; e < E; e += 64) {
-    const float v = expf(s[e] - mx);
-    s[e] = v;
-    sum += v;
-  }
-  sum = wave_sum(sum);
-  for (int e = lane; e < E; e += 64) {
-    const float v = s[e] / sum;
-    s[e] = v;
-    c[e] = v + (bias ? ld(bias + e) : 0.f);
-  }
-  const int per = E / G;
-  if (keep < G) {
-    for (int g = lane; g < G; g += 64) {
-      float best = -INFINITY;
-      for (int e = g * per; e < (g + 1) * per; ++e) best = fmaxf(best, c[e]);
-      gs[g] = best;
-    }
-    for (int g = lane; g < G; g += 64) {
-      const float mine = gs[g];
-      int better = 0;
-      for (int o2 = 0; o2 < G; ++o2) better += (gs[o2] > mine) || (gs[o2] == mine && o2 < g);
-      if (better >= keep)
-        for (int e = g * per; e < (g + 1) * per; ++e) c[e] = -INFINITY;
-    }
-  }
-  float tot = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float bv = -INFINITY;
-    int best = 0x7fffffff;
-    for (int e = lane; e < E; e += 64) {
-      const float v = c[e];
-      if (v > bv) {
-        bv = v;
-        best = e;
-      }
-    }
-#pragma unroll
-    for (int o = 32; o >= 1; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64);
-      const int oi = __shfl_xor(best, o, 64);
-      if (ov > bv || (ov == bv && oi < best)) {
-        bv = ov;
-        best = oi;
-      }
-    }
-    if (best == 0x7fffffff) best = 0;  // unreachable: the host checks top <= keep * (E / G) and choice scores are finite
-    const float sv = s[best];
-    tot += sv;
-    if (lane == 0) {
-      ids[k] = best;
-      gs[G + k] = sv;  // the chosen scores wait in LDS (in order within the wave) for the sum
-      c[best] = -INFINITY;
-    }
-  }
-  const float inv = 1.0f / (tot + 1e-20f);
-  for (int k = lane; k < top; k += 64) wts[k] = gs[G + k] * inv;
-}
-
+// so the matrix cores' fp32 accumulation IS the 32-bit router on the token's 16-bit copy); scores, choice and weights as in mix_route.h.
+// Scores live in LDS columns, one per thread.
 template <typename T>
 __global__ __launch_bounds__(64) void route_kernel(int* __restrict__ ids, float* __restrict__ wts, const float* __restrict__ z,
-                                                   const T* __restrict__ bias, int tokens, int E, int top, int G, int keep, int TPB) {
+                                                   const T* __restrict__ bias, int tokens, int E, int top, int G, int keep, RouteRule rule,
+                                                   int TPB) {
   extern __shared__ float lds[];
   const int t = blockIdx.x * TPB + threadIdx.x;
   if (threadIdx.x >= TPB || t >= tokens) return;
@@ -508,7 +379,7 @@ __global__ __launch_bounds__(64) void route_kernel(int* __restrict__ ids, float*
   const float* zr = z + (size_t)t * E;
 #pragma unroll 8
   for (int e = 0; e < E; ++e) s[e * TPB] = zr[e];
-  select_experts<T>(s, c, c + (size_t)E * TPB, TPB, bias, E, top, G, keep, ids + (size_t)t * top, wts + (size_t)t * top);
+  select_experts<T>(s, c, c + (size_t)E * TPB, TPB, bias, E, top, G, keep, rule, ids + (size_t)t * top, wts + (size_t)t * top);
 }
 
 template <typename T, bool ROUTE>
@@ -545,50 +416,10 @@ __global__ __launch_bounds__(256) void postnorm_kernel(const float* __restrict__
   if (!ROUTE) return;
   float* sc = red + 4;
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  // a wave takes experts wave, wave + 4, ...; up to kRouteAcc of them at once, so that one pass over the row has that many
-  // independent weight loads in flight per lane (element order per expert: lane-strided, then the wave reduction: fixed)
-  constexpr int kRouteAcc = 8;
-  const bool wide = (W & 7) == 0 && ((uintptr_t)router & 15u) == 0;
-  for (int e0 = wave; e0 < E; e0 += 4 * kRouteAcc) {
-    float acc[kRouteAcc];
-#pragma unroll
-    for (int a = 0; a < kRouteAcc; ++a) acc[a] = 0.f;
-    if (wide) {  // eight consecutive weights per lane and load: 16 bytes (bf16) or 32 (fp32)
-      for (int i = lane * 8; i < W; i += 512) {
-        float hv[8];
-#pragma unroll
-        for (int u = 0; u < 8; ++u) hv[u] = srow[i + u];
-#pragma unroll
-        for (int a = 0; a < kRouteAcc; ++a) {
-          const int e = e0 + 4 * a;
-          if (e < E) {
-            float wv[8];
-            read8(router + (size_t)e * W + i, wv);
-#pragma unroll
-            for (int u = 0; u < 8; ++u) acc[a] = fmaf(hv[u], wv[u], acc[a]);
-          }
-        }
-      }
-    } else {
-      for (int i = lane; i < W; i += 64) {
-        const float hv = srow[i];
-#pragma unroll
-        for (int a = 0; a < kRouteAcc; ++a) {
-          const int e = e0 + 4 * a;
-          if (e < E) acc[a] = fmaf(hv, ld(router + (size_t)e * W + i), acc[a]);
-        }
-      }
-    }
-#pragma unroll
-    for (int a = 0; a < kRouteAcc; ++a) {
-      const int e = e0 + 4 * a;
-      const float v = wave_sum(acc[a]);
-      if (e < E && lane == 0) sc[e] = v;
-    }
-  }
+  router_logits256(srow, router, E, W, sc);
   __syncthreads();
-  if (wave == 0) select_experts_wave<T>(sc, sc + E, sc + 2 * E, bias, E, top, G, keep, ids + (size_t)t * top, wts + (size_t)t * top);
+  if (threadIdx.x < 64)
+    select_experts_wave<T>(sc, sc + E, sc + 2 * E, bias, E, top, G, keep, RouteRule{0, 1, 1.0f}, ids + (size_t)t * top, wts + (size_t)t * top);
 }
 
 // ------------------------------------------------------------------------------------------------ expert bucketing
@@ -1244,11 +1075,12 @@ int msgl_mix_gated_norm(void* out, const float* o, const void* gate, int64_t ld_
   return MSGL_MIX_OK;
 }
 
-int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int tokens, int E, int top, int G, int keep, int dtype,
-                   void* stream) {
+int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int tokens, int E, int top, int G, int keep, int sigmoid,
+                   int group_best, float scale, int dtype, void* stream) {
   MIX_REQUIRE(ids && wts && z && dtype_ok(dtype), "route: null pointer / dtype");
   MIX_REQUIRE(E >= 1 && top >= 1 && top <= E && G >= 1 && E % G == 0 && keep >= 1 && keep <= G && top <= keep * (E / G),
               "route: bad sizes E %d top %d groups %d keep %d", E, top, G, keep);
+  MIX_REQUIRE(group_best == 1 || group_best == 2, "route: a group's score sums its 1 or 2 largest choices, not %d", group_best);
   if (tokens == 0) return MSGL_MIX_OK;
   int tpb = 64;
   while (tpb > 1 && (size_t)(2 * E + G) * tpb * sizeof(float) > 64 * 1024) tpb >>= 1;
@@ -1256,7 +1088,7 @@ int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int t
   MIX_REQUIRE(lds <= 64 * 1024, "route: too many experts");
   hipStream_t s = static_cast<hipStream_t>(stream);
   DISPATCH_T(dtype, hipLaunchKernelGGL(route_kernel<T>, dim3((tokens + tpb - 1) / tpb), dim3(64), lds, s, ids, wts, z, cp<T>(bias), tokens, E,
-                                       top, G, keep, tpb);)
+                                       top, G, keep, RouteRule{sigmoid, group_best, scale}, tpb);)
   MIX_LAUNCHED("route");
   return MSGL_MIX_OK;
 }

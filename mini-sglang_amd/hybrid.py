@@ -88,8 +88,21 @@ diff_attention     two softmax maps over the same values per head (q and k hold 
                    sequence.  Cached per token: k [G 2 d] and v [G dv].
 feed-forward       W_down of  g sigmoid(1.702 g) (u + 1),  g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit).
 
-Kernels: csrc/seqmix.hip, csrc/mix_delta.hip, csrc/mix_par.hip, csrc/mix_scan.hip and csrc/mix_streams.hip through mixops.py; plain projections through the library GEMM
-(mixops.linear).
+A sixth scheme, `sandwich` (the Redasun design): a norm on the way into every sublayer and another on its way out, and a loop that reads
+the embedding again at the start of every pass:
+
+stream             x_0 = s_e embed[token];  per layer  x <- x + n1b(mixer(n1(x))),  x <- x + n2b(ff(n2(x)));  n(v) = (v - mean) /
+                   sqrt(variance + eps) * w.  Layers start .. stop - 1 run `times` times in a row with the same weights, every pass with
+                   cache of its own, and before the first layer of every pass  x <- W_in [x; x_0].  Output: final norm, the embedding
+                   table itself as head matrix.
+diff_attention     as above without projection biases, gate and window: every earlier key is visible.
+feed-forward       W_down (gelu(W_gate h) * (W_up h)) with the tanh form of gelu, or routed experts W_down (silu(W_gate h) * (W_up h)):
+                   scores = sigmoid(router logits), choice = scores + a correction; of G groups of neighbours the `keep` best (by the
+                   sum of their two largest choices) can win, weights = the winners' scores over their sum, times a scale, on the
+                   experts' OUTPUTS; plus a shared expert that every token runs.
+
+Kernels: csrc/seqmix.hip, csrc/mix_delta.hip, csrc/mix_par.hip, csrc/mix_scan.hip, csrc/mix_streams.hip and csrc/mix_sandwich.hip through mixops.py;
+plain projections through the library GEMM (mixops.linear).
 """
 from __future__ import annotations
 
@@ -113,7 +126,10 @@ class MoeSpec:
     gated: bool = False             # expert = W_down (silu(W_gate h) * (W_up h)) instead of W_down relu(W_up h)^2
     pick: str = "scores"            # "scores": softmax over all experts, corrected group-limited choice; "logits": the largest
                                     # logits (+ bias) win and the weights are the softmax over the winners; "sigmoid_input": the
-                                    # largest logits win, weight = sigmoid(logit), and it multiplies the expert's INPUT
+                                    # largest logits win, weight = sigmoid(logit), and it multiplies the expert's INPUT;
+                                    # "sigmoid_scores": as "scores" with a sigmoid per expert in the place of the softmax
+    group_best: int = 1             # "scores", "sigmoid_scores": a group's score is the sum of its so many largest choices
+    scale: float = 1.0              # "sigmoid_scores": factor on the normalised weights
     shared_ff: int = 0              # inner size of a shared expert that every token runs (0: none)
 
 
@@ -123,13 +139,14 @@ class DenseFfSpec:
     act: str = "poly_norm"          # "poly_norm": c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3 with N = divide a row by its root mean square;
                                     # "xielu": softplus(p) z^2 + z / 2 above zero, (1/2 + softplus(q)) (exp(z) - 1 - z) + z / 2 below
                                     # "silu_gate": W_down (silu(W_gate h) * (W_up h))
+                                    # "gelu_gate": W_down (gelu(W_gate h) * (W_up h)), the tanh form of gelu
                                     # "clamp_gate": W_down (g sigmoid(slope g) (u + 1)), g = min(W_gate h, limit), u = W_up h within +-limit
     limit: float = 0.0              # clamp_gate
     slope: float = 1.702
 
     @property
     def gated(self) -> bool:
-        return self.act in ("silu_gate", "clamp_gate")
+        return self.act in ("silu_gate", "clamp_gate", "gelu_gate")
 
 
 @dataclass(frozen=True)
@@ -163,7 +180,8 @@ class LayerSpec:
     right: Optional["LayerSpec"] = None
     left_scale: float = 1.0
     right_scale: float = 1.0
-    out_gate: bool = False          # latent attention: the concatenated heads are multiplied by sigmoid(W_g h)
+    out_gate: bool = False          # latent, diff attention: the concatenated heads are multiplied by sigmoid(W_g h)
+    proj_bias: bool = False         # diff_attention: the q, k, v projections have biases
     v_norm: bool = False            # sink attention: every value head is divided by its root mean square before it is cached
     dt_rank: int = 0                # mamba1: inner size of the two-step step-size projection
     maps: int = 1                   # diff_attention: 2, the softmax maps whose difference a head is
@@ -192,7 +210,7 @@ class HybridConfig:
     residual: str = "post_norm"     # "post_norm": x <- norm(alpha x + f(x)), weights stored as offsets from one, tied head;
                                     # "pre_norm_depth": x + f(norm(x)), depth-averaged history, normed embedding, own head;
                                     # "parallel_shift": x + ls1 mixer(shift(norm(x))) + ls2 ff(norm(x)), own head
-    embed_scale: float = 1.0        # parallel_shift: the embedding row is multiplied by this
+    embed_scale: float = 1.0        # parallel_shift, sandwich: the embedding row is multiplied by this
     pair_embed: Optional[Tuple[int, int, int]] = None  # (buckets, multiplier of the previous id, multiplier of the id) of the pair table
     token_shift: bool = False       # every layer's mixer reads a blend of this token's and the previous token's normed row
     # "pre_norm_conv": x + m f(conv(norm(x))), norms in groups, a looped run of layers, capped logits, own head
@@ -204,6 +222,8 @@ class HybridConfig:
     # "streams": several residual streams joined by small matrices around every sublayer, tanh in the place of norms, own head
     streams: int = 1
     logit_scale: float = 1.0        # logits <- scale * head x
+    # "sandwich": x + n'(f(n(x))), tied head; with a loop every pass starts from loop_in [x; embedding]
+    norm_centre: bool = False       # norms take the row's mean off first
 
     @property
     def num_layers(self) -> int:
@@ -440,7 +460,7 @@ def nagezen_config(cfg: Dict[str, Any], shapes: Optional[Dict[str, Tuple[int, ..
             sc = (m.get("rot") or {}).get("scaling")
             if H % G:
                 raise ValueError(f"layer {i}: {H} heads over {G} key heads")
-            layers.append(LayerSpec(kind="diff_attention", heads=H, kv_heads=G, dim=d, vdim=dv, scale=float(m["scale"]), maps=2,
+            layers.append(LayerSpec(kind="diff_attention", heads=H, kv_heads=G, dim=d, vdim=dv, scale=float(m["scale"]), maps=2, proj_bias=True,
                                     window=int(mask.get("size", 0)), keep_first=int(mask.get("keep_first", 0)), diff=float(m["diff"]),
                                     rot_dims=dims, rot_base=base,
                                     rot_scaling=None if not sc else tuple(sorted((k, float(v)) for k, v in sc.items())), out_gate=True, mlp=ff))
@@ -451,6 +471,44 @@ def nagezen_config(cfg: Dict[str, Any], shapes: Optional[Dict[str, Tuple[int, ..
         raise ValueError(f"{streams} residual streams")
     return HybridConfig(vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]), layers=tuple(layers), rms_norm_eps=float(cfg["norm"]["eps"]),
                         name=name, residual="streams", streams=streams, logit_scale=float(cfg.get("logit_scale", 1.0)))
+
+
+def redasun_config(cfg: Dict[str, Any], name: str = "Redasun") -> HybridConfig:
+    """config.json of a Redasun model -> HybridConfig."""
+    layers: List[LayerSpec] = []
+    for i, entry in enumerate(cfg["layers"]):
+        m, kind, mlp = entry["mixer"], entry["type"], entry.get("mlp")
+        if kind != "attention":
+            raise ValueError(f"layer {i}: unknown mixer type {kind!r}")
+        ff = None
+        if mlp is not None:
+            if mlp.get("kind") == "dense":
+                ff = DenseFfSpec(ff=int(mlp["ff"]), act="gelu_gate")
+            elif mlp.get("kind") == "moe":
+                r, sh = mlp["router"], mlp.get("shared")
+                g = r.get("groups") or {}
+                count = int(g.get("count", 1))
+                ff = MoeSpec(experts=int(r["experts"]), top=int(r["top"]), ff=int(mlp["expert"]["ff"]), groups=count, keep=int(g.get("keep", count)),
+                             gated=True, pick="sigmoid_scores", group_best=2, scale=float(r.get("scale", 1.0)), shared_ff=int(sh["ff"]) if sh else 0)
+                if ff.experts % count or not 1 <= ff.keep <= count or not 1 <= ff.top <= ff.keep * (ff.experts // count):
+                    raise ValueError(f"layer {i}: top {ff.top} of {ff.experts} experts in the best {ff.keep} of {count} groups")
+            else:
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp.get('kind')!r}")
+        H, d = int(m["heads"]), int(m["dim"])
+        G = int(m.get("kv_heads", H))
+        dims, base = _rot(m, 0)
+        if H % G or dims % 2 or dims > d:
+            raise ValueError(f"layer {i}: {H} heads over {G} key heads, a rotation of {dims} entries in heads of {d}")
+        layers.append(LayerSpec(kind="diff_attention", heads=H, kv_heads=G, dim=d, vdim=int(m["vdim"]), scale=float(m["scale"]), maps=2,
+                                diff=float(m["diff"]), rot_dims=dims, rot_base=base, mlp=ff))
+    loop = cfg.get("loop")
+    lp = None
+    if loop:
+        lp = (int(loop["start"]), int(loop["stop"]), int(loop["times"]))
+        if not (0 <= lp[0] < lp[1] <= len(layers) and lp[2] >= 1):
+            raise ValueError(f"loop {lp} over {len(layers)} layers")
+    return HybridConfig(vocab_size=int(cfg["vocab"]), hidden_size=int(cfg["width"]), layers=tuple(layers), rms_norm_eps=float(cfg["norm"]["eps"]),
+                        name=name, residual="sandwich", norm_centre=True, loop=lp, embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)))
 
 
 def wavelength_scaled_rotary_table(dims: int, base: float, scaling: Optional[Dict[str, float]], max_position: int, device) -> torch.Tensor:
@@ -488,7 +546,7 @@ class _Layer:
     __slots__ = ("spec", "w_in", "o", "norm1", "norm2", "uk_t", "uv", "c_norm", "cos_sin", "out_norm", "decay", "router",
                  "bias", "up", "down", "talk", "lam", "taps", "rate", "dt_bias", "a2", "g2", "act", "depth_w",
                  "sink", "ls1", "ls2", "shift", "in_bias", "out_bias", "pb", "skip", "conv_b", "sum_bias", "canon1", "canon2", "w_x", "w_dt",
-                 "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k", "lam_now", "sq1", "sq2", "hc1", "hc2")
+                 "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k", "lam_now", "sq1", "sq2", "hc1", "hc2", "norm1b", "norm2b")
 
     def __init__(self, spec: LayerSpec) -> None:
         self.spec = spec
@@ -539,8 +597,9 @@ class HybridDecoder:
         self.parallel = cfg.residual == "parallel_shift"
         self.conv_stream = cfg.residual == "pre_norm_conv"
         self.multi = cfg.residual == "streams"
+        self.sandwich = cfg.residual == "sandwich"
         self.final_squash: Optional[_Squash] = None
-        self.embed_norm = self.head = self.pair_table = self.loop_step = None
+        self.embed_norm = self.head = self.pair_table = self.loop_step = self.loop_in = None  # head None: the embedding table
         self.embed = w(cfg.vocab_size, W, std=1.0)
         self.final_norm = None if self.multi else w(W, std=0.1)
         self.layers: List[_Layer] = []
@@ -602,13 +661,15 @@ class HybridDecoder:
                     L.cos_sin = plain_table(spec.rot_dims, spec.rot_base) if spec.rot_dims else None
             elif spec.kind == "diff_attention":
                 G, n = spec.kv_heads, (H + spec.kv_heads) * spec.maps * d + spec.kv_heads * dv
-                L.w_in = w(n + H * dv, W, std=W ** -0.5)  # q | k | v | gate
-                L.in_bias = f32(n, std=0.1)
+                L.w_in = w(n + (H * dv if spec.out_gate else 0), W, std=W ** -0.5)  # q | k | v (| gate)
+                L.in_bias = f32(n, std=0.1) if spec.proj_bias else None
                 L.q_norm, L.k_norm = (1.0 + w(d, std=0.1).float()).to(dtype), (1.0 + w(d, std=0.1).float()).to(dtype)
                 L.lam_q, L.lam_k = f32(spec.maps, d, std=0.1), f32(spec.maps, d, std=0.1)
                 L.lam_now = f32(1)
                 L.o = w(W, H * dv, std=(H * dv) ** -0.5)
-                if spec.rot_dims:
+                if spec.rot_dims and spec.rot_scaling is None:
+                    L.cos_sin = plain_table(spec.rot_dims, spec.rot_base)
+                elif spec.rot_dims:
                     key = (spec.rot_dims, spec.rot_base, spec.rot_scaling)
                     if key not in tables:
                         tables[key] = rotary_table(spec, self.max_position, device)
@@ -688,6 +749,10 @@ class HybridDecoder:
             if isinstance(m, MoeSpec) and m.shared_ff:
                 L.sh_up = w(2 * m.shared_ff, W, std=W ** -0.5)
                 L.sh_down = w(W, m.shared_ff, std=m.shared_ff ** -0.5)
+            if self.sandwich:
+                L.norm1, L.norm1b = (1.0 + L.norm1.float()).to(dtype), (1.0 + w(W, std=0.1).float()).to(dtype)
+                if m is not None:
+                    L.norm2, L.norm2b = (1.0 + L.norm2.float()).to(dtype), (1.0 + w(W, std=0.1).float()).to(dtype)
             if self.conv_stream:
                 L.norm1, L.norm2 = (1.0 + L.norm1.float()).to(dtype), None if L.norm2 is None else (1.0 + L.norm2.float()).to(dtype)
                 if cfg.conv_taps:
@@ -708,6 +773,11 @@ class HybridDecoder:
             self.head = w(cfg.vocab_size, W, std=W ** -0.5)
             if cfg.loop is not None:
                 self.loop_step = f32(cfg.loop[2], W, std=0.3)
+        if self.sandwich:
+            self.final_norm = (1.0 + self.final_norm.float()).to(dtype)
+            if cfg.loop is not None:
+                self.loop_in = w(W, 2 * W, std=(2 * W) ** -0.5)
+            self._derive()
         if self.multi:
             self.final_squash = squash()
             self.head = w(cfg.vocab_size, W, std=W ** -0.5)
@@ -733,13 +803,13 @@ class HybridDecoder:
 
     def _tensors(self):
         yield self.embed
-        for t in (self.final_norm, self.embed_norm, self.head, self.pair_table, self.loop_step):
+        for t in (self.final_norm, self.embed_norm, self.head, self.pair_table, self.loop_step, self.loop_in):
             if t is not None:
                 yield t
         for L in self.layers:
             for k in ("w_in", "o", "norm1", "norm2", "uk_t", "uv", "c_norm", "out_norm", "router", "bias", "up", "down", "talk", "lam",
                       "taps", "rate", "dt_bias", "a2", "g2", "act", "depth_w", "sink", "ls1", "ls2", "shift", "in_bias", "out_bias", "pb",
-                      "skip", "conv_b", "canon1", "canon2", "w_x", "w_dt", "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k"):
+                      "skip", "conv_b", "canon1", "canon2", "w_x", "w_dt", "sh_up", "sh_down", "q_norm", "k_norm", "lam_q", "lam_k", "norm1b", "norm2b"):
                 t = getattr(L, k)
                 if t is not None:
                     yield t
@@ -796,6 +866,8 @@ class HybridDecoder:
             put(self.head, state["head"])
             if self.loop_step is not None:
                 put(self.loop_step, state["loop.step"])
+        if self.loop_in is not None:
+            put(self.loop_in, state["loop.in"])
         for i, L in enumerate(self.layers):
             s, p = L.spec, f"l{i}.mix."
             H, d, dv = s.heads, s.dim, s.vdim
@@ -807,6 +879,10 @@ class HybridDecoder:
                     put_junction(L.hc2, f"l{i}.hc2")
             else:
                 put(L.norm1, state[f"l{i}.norm1"])
+            if L.norm1b is not None:
+                put(L.norm1b, state[f"l{i}.norm1b"])
+            if L.norm2b is not None:
+                put(L.norm2b, state[f"l{i}.norm2b"])
             if L.canon1 is not None:
                 put(L.canon1, state[f"l{i}.canon1"])
             if L.canon2 is not None:
@@ -841,8 +917,9 @@ class HybridDecoder:
                     put(L.dt_bias, state[p + "a2.b"])
                     put(L.out_norm, state[p + "norm"])
             elif s.kind == "diff_attention":
-                put(L.w_in, torch.cat([state[p + n] for n in ("q", "k", "v", "g")], dim=0))
-                put(L.in_bias, torch.cat([state[p + n + ".b"] for n in ("q", "k", "v")], dim=0))
+                put(L.w_in, torch.cat([state[p + n] for n in ("q", "k", "v") + (("g",) if s.out_gate else ())], dim=0))
+                if L.in_bias is not None:
+                    put(L.in_bias, torch.cat([state[p + n + ".b"] for n in ("q", "k", "v")], dim=0))
                 put(L.q_norm, state[p + "q.norm"])
                 put(L.k_norm, state[p + "k.norm"])
                 put(L.lam_q, torch.stack([state[p + "lq1"], state[p + "lq2"]]))
@@ -885,7 +962,7 @@ class HybridDecoder:
             if s.kind != "parallel":
                 put(L.o, state[p + "o"])
             if s.mlp is None and f"l{i}.norm2" in state and not self.pre_norm and not self.parallel and not self.conv_stream and \
-                    not self.multi:  # no feed-forward, but a second norm
+                    not self.multi and not self.sandwich:  # no feed-forward, but a second norm
                 L.norm2 = torch.empty_like(L.norm1)
                 put(L.norm2, state[f"l{i}.norm2"])
             if isinstance(s.mlp, DenseFfSpec) and s.mlp.gated:
@@ -907,6 +984,11 @@ class HybridDecoder:
                 put(L.router, state[q + "router"])
                 if s.mlp.pick == "sigmoid_input":
                     L.bias = None
+                    if s.mlp.shared_ff:
+                        put(L.sh_up, torch.cat([state[q + "shared.gate"], state[q + "shared.up"]], dim=0))
+                        put(L.sh_down, state[q + "shared.down"])
+                elif s.mlp.pick == "sigmoid_scores":
+                    put(L.bias, state[q + "correction"])
                     if s.mlp.shared_ff:
                         put(L.sh_up, torch.cat([state[q + "shared.gate"], state[q + "shared.up"]], dim=0))
                         put(L.sh_down, state[q + "shared.down"])
@@ -944,6 +1026,8 @@ class HybridDecoder:
             out["head"] = self.head
             if self.loop_step is not None:
                 out["loop.step"] = self.loop_step
+        if self.loop_in is not None:
+            out["loop.in"] = self.loop_in
         for i, L in enumerate(self.layers):
             s, p = L.spec, f"l{i}.mix."
             H, d, dv = s.heads, s.dim, s.vdim
@@ -954,6 +1038,10 @@ class HybridDecoder:
                     out[j + ".in"], out[j + ".out"], out[j + ".mix"] = hc.read, hc.out, hc.mix
             if not self.multi:
                 out[f"l{i}.norm1"] = L.norm1
+            if L.norm1b is not None:
+                out[f"l{i}.norm1b"] = L.norm1b
+            if L.norm2b is not None:
+                out[f"l{i}.norm2b"] = L.norm2b
             if L.canon1 is not None:
                 out[f"l{i}.canon1"] = L.canon1
             if L.canon2 is not None:
@@ -987,10 +1075,11 @@ class HybridDecoder:
                     out[p + n] = t
             elif s.kind == "diff_attention":
                 cuts = [H * s.maps * d, s.kv_heads * s.maps * d, s.kv_heads * dv]
-                for n, t in zip(("q", "k", "v", "g"), torch.split(L.w_in, cuts + [H * dv], dim=0)):
+                for n, t in zip(("q", "k", "v", "g"), torch.split(L.w_in, cuts + ([H * dv] if s.out_gate else []), dim=0)):
                     out[p + n] = t
-                for n, t in zip(("q", "k", "v"), torch.split(L.in_bias, cuts, dim=0)):
-                    out[p + n + ".b"] = t
+                if L.in_bias is not None:
+                    for n, t in zip(("q", "k", "v"), torch.split(L.in_bias, cuts, dim=0)):
+                        out[p + n + ".b"] = t
                 out[p + "q.norm"], out[p + "k.norm"] = L.q_norm, L.k_norm
                 for a in range(s.maps):
                     out[p + f"lq{a + 1}"], out[p + f"lk{a + 1}"] = L.lam_q[a], L.lam_k[a]
@@ -1043,7 +1132,9 @@ class HybridDecoder:
             elif isinstance(s.mlp, MoeSpec) and s.mlp.gated:
                 q = f"l{i}.mlp."
                 out[f"l{i}.norm2"], out[q + "router"] = L.norm2, L.router
-                if s.mlp.pick == "sigmoid_input":
+                if s.mlp.pick == "sigmoid_scores":
+                    out[q + "correction"] = L.bias
+                if s.mlp.pick in ("sigmoid_input", "sigmoid_scores"):
                     if s.mlp.shared_ff:
                         out[q + "shared.gate"], out[q + "shared.up"] = L.sh_up[: s.mlp.shared_ff], L.sh_up[s.mlp.shared_ff:]
                         out[q + "shared.down"] = L.sh_down
@@ -1218,10 +1309,81 @@ class HybridDecoder:
         q = mixops.qk_prep(proj, L.in_bias, kc, vc, batch.out_loc, batch.positions, L.cos_sin, eps, H * M, G * M, d, dv, interleaved=False,
                            unit=False, norm_w=(L.q_norm, L.k_norm), value_heads=G)
         o = torch.empty((T, H * dv), dtype=self.dtype, device=h.device)
+        gate = proj[:, L.w_in.shape[0] - H * dv:] if s.out_gate else None
         splits = mixops.sink_attn_splits(md.batch, T, H, G, s.window, md.max_seqlen_k, s.keep_first) if md.max_seqlen_q <= 16 else 1
         mixops.diff_attn(o, q, kc, vc, ctx.page_table, md.req_rows, md.seq_lens, md.cu_seqlens_q, md.batch, H, G, d, dv, s.scale, s.window,
-                         s.keep_first, L.lam_now, 1.0 - s.diff, eps, gate=proj[:, L.in_bias.shape[0]:], splits=splits)
+                         s.keep_first, L.lam_now, 1.0 - s.diff, eps, gate=gate, splits=splits)
         return mixops.linear(o, L.o)
+
+    def _gated_ff_act(self, h: torch.Tensor, up: torch.Tensor, down: torch.Tensor, act: int) -> torch.Tensor:
+        return mixops.linear(mixops.gate_mul(mixops.linear(h, up), act), down)
+
+    def _forward_sandwich(self, ctx: Any, batch: Any, layer_outputs: Optional[list]) -> torch.Tensor:
+        """The stream with a norm into and out of every sublayer -> the final-normed rows [tokens, W].  One `join_norm` launch closes a
+        sublayer (weighted sum of its outputs, their norm, the residual sum) and opens the next (norm; in short batches also the router's
+        choice); at the start of a pass of the loop it leaves the stream as product rows beside the embedding's instead, and the fp32
+        product of the two is the new stream."""
+        cfg = self.cfg
+        T, W, dev = batch.input_ids.shape[0], cfg.hidden_size, self.device
+        x = torch.empty((T, W), dtype=torch.float32, device=dev)
+        join = dict(dtype=self.dtype, centre=cfg.norm_centre)
+        both = torch.empty((T, 2 * W), dtype=self.dtype, device=dev) if self.loop_in is not None else None  # rows [x | embedding]
+        runs = cfg.runs
+        state: Dict[str, Any] = dict(src=None, close={})  # close: what the sublayer before left to be summed
+
+        def step(w_out=None, h_out=None, raw=(), route=None):
+            """Closes the sublayer before (or reads the embedding rows) and writes what is asked for."""
+            kw, out = state["close"], x
+            if state["src"] is None:
+                kw = dict(embed=(self.embed, batch.input_ids, cfg.embed_scale))
+                if both is not None:
+                    raw = tuple(raw) + (both[:, W:],)
+            elif not kw:
+                out = None  # the stream is in x already
+            picks = mixops.join_norm(state["src"], cfg.rms_norm_eps, x_out=out, raw=raw, w_out=w_out, h_out=h_out, route=route, **join, **kw)
+            state.update(src=x, close={})
+            return picks
+
+        def row():
+            return torch.empty((T, W), dtype=self.dtype, device=dev)
+
+        for run, (i, pass_no) in enumerate(runs):
+            L = self.layers[i]
+            m = L.spec.mlp
+            if pass_no is not None:
+                step(raw=(both[:, :W],))
+                if layer_outputs is not None and run > 0:
+                    layer_outputs.append(x.clone())
+                mixops.linear(both, self.loop_in, out=x)
+            h = row()
+            step(w_out=L.norm1, h_out=h)
+            if layer_outputs is not None and run > 0 and pass_no is None:
+                layer_outputs.append(x.clone())
+            if L.spec.kind != "diff_attention":
+                raise NotImplementedError(f"mixer {L.spec.kind!r} in a sandwich-norm stack")
+            state["close"] = dict(y=self._diff_attention(run, L, h, ctx, batch), w_in=L.norm1b)
+            if m is None:
+                continue
+            h = row()
+            if isinstance(m, DenseFfSpec):
+                step(w_out=L.norm2, h_out=h)
+                state["close"] = dict(y=self._gated_ff_act(h, L.up, L.down, mixops.GATE_MUL_GELU_TANH), w_in=L.norm2b)
+                continue
+            # few tokens: the norm's launch also routes; many: every token re-reading the router matrix costs more than the launches
+            # it saves, so the logits come from the product kernel
+            fuse = T <= self.ROUTE_FUSE_MAX_TOKENS
+            rule = (m.top, m.groups, m.keep, True, m.group_best, m.scale)
+            picks = step(w_out=L.norm2, h_out=h, route=(L.router, L.bias) + rule if fuse else None)
+            if not fuse:
+                picks = mixops.route(h, L.router, L.bias, m.top, m.groups, m.keep, sigmoid=True, group_best=m.group_best, scale=m.scale)
+            y = self._gated_experts(L, h, picks[0])
+            y2 = self._gated_ff_act(h, L.sh_up, L.sh_down, mixops.GATE_MUL_SILU) if m.shared_ff else None
+            state["close"] = dict(y=y, gate=picks[1], y2=y2, w_in=L.norm2b)
+        hf = row()
+        step(w_out=self.final_norm, h_out=hf)
+        if layer_outputs is not None and runs:
+            layer_outputs.append(x.clone())
+        return hf
 
     def _forward_streams(self, ctx: Any, batch: Any, layer_outputs: Optional[list]) -> torch.Tensor:
         """Several residual streams -> the rows in front of the LM head [tokens, W].  One `stream_norm` launch closes a sublayer (all
@@ -1448,8 +1610,8 @@ class HybridDecoder:
         last token (prefill) or at every token (decode)."""
         cfg = self.cfg
         eps, alpha = cfg.rms_norm_eps, cfg.postln_alpha
-        if self.pre_norm or self.parallel or self.conv_stream or self.multi:
-            run = self._forward_pre_norm if self.pre_norm else self._forward_parallel if self.parallel else \
+        if self.pre_norm or self.parallel or self.conv_stream or self.multi or self.sandwich:
+            run = self._forward_sandwich if self.sandwich else self._forward_pre_norm if self.pre_norm else self._forward_parallel if self.parallel else \
                 self._forward_conv if self.conv_stream else self._forward_streams
             hf = run(ctx, batch, layer_outputs)
             rows = getattr(batch, "logit_rows", None)
@@ -1457,10 +1619,11 @@ class HybridDecoder:
                 rows = batch.attn_metadata.get_last_indices(batch.size)
             if rows is not None:
                 hf = hf.index_select(0, rows.to(torch.int64))
+            head = self.embed if self.head is None else self.head
             if logits_out is not None and logits_out.shape == (hf.shape[0], cfg.vocab_size) and logits_out.dtype == self.dtype:
-                logits = mixops.linear(hf, self.head, out=logits_out)
+                logits = mixops.linear(hf, head, out=logits_out)
             else:
-                logits = mixops.linear(hf, self.head)
+                logits = mixops.linear(hf, head)
             return mixops.softcap(logits, cfg.logit_softcap) if cfg.logit_softcap > 0.0 else logits
         x, h = mixops.embed(self.embed, batch.input_ids)
         for i, L in enumerate(self.layers):

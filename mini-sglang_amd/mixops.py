@@ -170,9 +170,11 @@ def gated_norm(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, eps: f
     return out
 
 
-def route(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int, groups: int, keep: int):
+def route(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int, groups: int, keep: int, *, sigmoid: bool = False,
+          group_best: int = 1, scale: float = 1.0):
     """-> (expert ids int32 [T, top], weights fp32 [T, top]).  Router logits in fp32 (fp32 accumulation over the token's copy in
-    the model dtype: 16-bit products are exact in fp32), then softmax, corrected group-limited choice and weights in one pass."""
+    the model dtype: 16-bit products are exact in fp32), then softmax (or a sigmoid per expert), corrected group-limited choice (a
+    group's score: the sum of its `group_best` largest choices) and weights (times scale) in one pass."""
     _dev(h, router, bias)
     T, W = h.shape
     E = router.shape[0]
@@ -182,8 +184,8 @@ def route(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], t
     gemm_nt(z, h, router, T, E, W, lda=W, ldb=W, ldc=E)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=h.device)
-    check_mix(mix_lib().msgl_mix_route(ids.data_ptr(), wts.data_ptr(), z.data_ptr(), _p(bias), T, E, top, groups, keep, _code(h),
-                                       _stream()), "route")
+    check_mix(mix_lib().msgl_mix_route(ids.data_ptr(), wts.data_ptr(), z.data_ptr(), _p(bias), T, E, top, groups, keep, int(sigmoid),
+                                       int(group_best), float(scale), _code(h), _stream()), "route")
     return ids, wts
 
 
@@ -213,7 +215,8 @@ _NO_LIBRARY_SOLUTION: set = set()
 
 
 def linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[M, N] = x[M, K] w[N, K]^T, fp32 accumulation, output in x's dtype."""
+    """out[M, N] = x[M, K] w[N, K]^T, fp32 accumulation, output in x's dtype (or, for 16-bit operands, into an fp32 `out`: a product that
+    is the residual stream itself)."""
     _dev(x, w)
     assert x.dim() == 2 and w.dim() == 2 and x.shape[1] == w.shape[1] and x.dtype == w.dtype
     assert x.stride(1) == 1 and w.stride(1) == 1
@@ -223,14 +226,16 @@ def linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None)
         out = torch.empty((M, N), dtype=x.dtype, device=x.device)
     if M == 0:
         return out
-    key = (M, N, K, x.stride(0), w.stride(0), out.stride(0), x.dtype)
+    assert out.dtype in (x.dtype, torch.float32) and out.shape == (M, N) and out.stride(1) == 1
+    key = (M, N, K, x.stride(0), w.stride(0), out.stride(0), x.dtype, out.dtype)
     if key not in _NO_LIBRARY_SOLUTION:
         try:
-            if x.dtype == torch.float32:
+            if out.dtype == torch.float32:
                 ws = ops.gemm_workspace(x.device)
+                code = _lib.F32 if x.dtype == torch.float32 else _lib.BF16_OUT_F32
                 _lib.check_gemm(_lib.gemm_lib().msgl_gemm_nt(
-                    out.data_ptr(), x.data_ptr(), w.data_ptr(), M, N, K, x.stride(0), w.stride(0), out.stride(0), _lib.F32,
-                    ws.data_ptr(), ws.numel(), _stream()), "gemm_nt (fp32)")
+                    out.data_ptr(), x.data_ptr(), w.data_ptr(), M, N, K, x.stride(0), w.stride(0), out.stride(0), code,
+                    ws.data_ptr(), ws.numel(), _stream()), "gemm_nt (fp32 result)")
                 return out
             return ops.linear(x, w, out=out)
         except _lib.MsglError:
@@ -241,6 +246,7 @@ def linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None)
 
 # ------------------------------------------------------------------ pre-norm hybrid decoders (csrc/mix_delta.hip)
 GATE_SIGMOID, GATE_SILU = 0, 1
+GATE_MUL_SILU, GATE_MUL_GELU_TANH = 0, 1
 
 
 def embed_norm(table: torch.Tensor, ids: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor) -> torch.Tensor:
@@ -315,12 +321,7 @@ def poly_act(z: torch.Tensor, coef: torch.Tensor, eps: float) -> torch.Tensor:
 
 def silu_mul(gate_up: torch.Tensor) -> torch.Tensor:
     """rows [gate | up] of 2 N -> silu(gate) * up, rows of N."""
-    _dev(gate_up)
-    rows, N2 = gate_up.shape
-    assert gate_up.is_contiguous() and N2 % 2 == 0
-    out = torch.empty((rows, N2 // 2), dtype=gate_up.dtype, device=gate_up.device)
-    check_mix(mix_lib().msgl_mix_silu_mul(out.data_ptr(), gate_up.data_ptr(), rows, N2 // 2, _code(gate_up), _stream()), "silu_mul")
-    return out
+    return gate_mul(gate_up, GATE_MUL_SILU)
 
 
 def route_top(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int):
@@ -886,4 +887,67 @@ def clamp_gate(gu: torch.Tensor, limit: float, slope: float) -> torch.Tensor:
     assert gu.is_contiguous() and gu.shape == (rows, 2 * N)
     out = torch.empty((rows, N), dtype=gu.dtype, device=gu.device)
     check_mix(mix_lib().msgl_mix_clamp_gate(out.data_ptr(), gu.data_ptr(), rows, N, float(limit), float(slope), _code(gu), _stream()), "clamp_gate")
+    return out
+
+
+# ------------------------------------------------------------------ decoders that norm a sublayer's input and output (csrc/mix_sandwich.hip)
+def join_norm(x: Optional[torch.Tensor], eps: float, *, dtype: torch.dtype, centre: bool, embed=None, y: Optional[torch.Tensor] = None,
+              gate: Optional[torch.Tensor] = None, y2: Optional[torch.Tensor] = None, w_in: Optional[torch.Tensor] = None,
+              x_out: Optional[torch.Tensor] = None, raw=(), w_out: Optional[torch.Tensor] = None, h_out: Optional[torch.Tensor] = None, route=None):
+    """x' = x + N(sum_p gate[:, p] y[:, p] + y2) * w_in -> x_out (fp32, may be x);  h = N(x') * w_out -> h_out;  N = rms_unit, after the
+    row's mean is taken off with `centre`.  x: fp32 [rows, W], or None with embed = (table [V, W], ids, scale): scaled embedding rows.
+    y: [rows, W] or [rows, p, W], gate fp32 [rows, p] or None, y2 [rows, W]; w_in None: the sum is added as it is.  raw: up to two
+    [rows, W] views in `dtype` with a common row stride that get x' too.  route = (router [E, W], bias [E] | None, top, groups, keep,
+    sigmoid, group_best, scale): h is routed in the same launch -> (expert ids int32 [rows, top], weights fp32 [rows, top])."""
+    table = ids = None
+    scale = 1.0
+    if x is None:
+        table, ids, scale = embed
+        _dev(table, ids)
+        assert table.dim() == 2 and table.is_contiguous() and table.dtype == dtype
+        rows, W = ids.shape[0], table.shape[1]
+    else:
+        rows, W = x.shape
+        assert embed is None and x.dtype == torch.float32 and x.is_contiguous()
+    _dev(x, y, gate, y2, w_in, x_out, w_out, h_out, *raw)
+    parts = 0
+    if y is not None:
+        assert y.dtype == dtype and y.is_contiguous() and y.shape[0] == rows and y.shape[-1] == W and y.dim() in (2, 3)
+        parts = 1 if y.dim() == 2 else y.shape[1]
+    assert gate is None or (y is not None and gate.dtype == torch.float32 and gate.is_contiguous() and gate.numel() == rows * parts)
+    for t in (y2, h_out):
+        assert t is None or (t.dtype == dtype and t.is_contiguous() and t.shape == (rows, W))
+    for t in (w_in, w_out):
+        assert t is None or (t.dtype == dtype and t.is_contiguous() and t.shape == (W,))
+    assert x_out is None or (x_out.dtype == torch.float32 and x_out.is_contiguous() and x_out.shape == (rows, W))
+    raw = tuple(raw)
+    assert len(raw) <= 2 and all(t.dtype == dtype and t.shape == (rows, W) and t.stride(1) == 1 and t.stride(0) == raw[0].stride(0) for t in raw)
+    router = bias = pick = wts = None
+    E = top = groups = keep = sigmoid = group_best = 0
+    rscale = 1.0
+    if route is not None:
+        router, bias, top, groups, keep, sigmoid, group_best, rscale = route
+        _dev(router, bias)
+        E = router.shape[0]
+        assert router.shape == (E, W) and router.is_contiguous() and router.dtype == dtype
+        assert bias is None or (bias.dtype == dtype and bias.shape == (E,) and bias.is_contiguous())
+        dev = router.device
+        pick = torch.empty((rows, top), dtype=torch.int32, device=dev)
+        wts = torch.empty((rows, top), dtype=torch.float32, device=dev)
+    if rows:
+        check_mix(mix_lib().msgl_mix_join_norm(
+            _p(x), _p(table), _p(None if ids is None else _i32(ids)), float(scale), _p(y), parts, _p(gate), _p(y2), _p(w_in), _p(x_out),
+            _p(raw[0]) if raw else 0, _p(raw[1]) if len(raw) > 1 else 0, raw[0].stride(0) if raw else 0, _p(w_out), _p(h_out), float(eps),
+            int(centre), rows, W, _lib.BF16 if dtype == torch.bfloat16 else _lib.F32, _p(router), _p(bias), E, top, groups, keep, int(sigmoid),
+            int(group_best), float(rscale), _p(pick), _p(wts), _stream()), "join_norm")
+    return None if route is None else (pick, wts)
+
+
+def gate_mul(gu: torch.Tensor, act: int) -> torch.Tensor:
+    """gu [rows, 2 N] = gate | up -> act(gate) * up, act = GATE_MUL_SILU or GATE_MUL_GELU_TANH."""
+    _dev(gu)
+    rows, N = gu.shape[0], gu.shape[1] // 2
+    assert gu.is_contiguous() and gu.shape == (rows, 2 * N)
+    out = torch.empty((rows, N), dtype=gu.dtype, device=gu.device)
+    check_mix(mix_lib().msgl_mix_gate_mul(out.data_ptr(), gu.data_ptr(), rows, N, int(act), _code(gu), _stream()), "gate_mul")
     return out

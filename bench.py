@@ -687,7 +687,17 @@ def main() -> None:
                          "linear attention, two-map windowed attention) beside the looped pre-norm hybrid decoder of equal size, and its "
                          "kernels against their rooflines (tools/nagezen_bench.py; further flags after --nagezen-args)")
     ap.add_argument("--nagezen-args", nargs=argparse.REMAINDER, default=[], help="flags handed to tools/nagezen_bench.py")
+    ap.add_argument("--redasun", action="store_true",
+                    help="instead of the default workload: prefill / decode throughput of the looped sandwich-norm decoder (two-map attention, "
+                         "group-limited sigmoid router with a shared expert) beside the looped pre-norm hybrid decoder of equal size, and its "
+                         "kernels against their rooflines (tools/redasun_bench.py; further flags after --redasun-args)")
+    ap.add_argument("--redasun-args", nargs=argparse.REMAINDER, default=[], help="flags handed to tools/redasun_bench.py")
     args = ap.parse_args()
+    if args.redasun:
+        from tools.redasun_bench import main as redasun_main
+
+        redasun_main(list(args.redasun_args))
+        return
     if args.nagezen:
         from tools.nagezen_bench import main as nagezen_main
 

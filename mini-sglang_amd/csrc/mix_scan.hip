@@ -431,7 +431,7 @@ __global__ __launch_bounds__(256) void selective_join_kernel(const float* __rest
 // A workgroup = 16 query rows (QT tokens of one request x HB query heads of ONE key/value head) x 16 lanes, one range of the
 // visible keys.  splits > 1: (max, sum, unnormalised output) per range, joined by sink_merge_kernel, where the sink enters.
 constexpr int kSinkRows = 16;
-constexpr int kSinkMaxC = 16;  // value columns per lane: dv <= 256
+constexpr int kSinkMaxDv = 1024;
 
 struct DiffOut {  // what two maps become one output row with
   const float* lam;  // one number on the device
@@ -440,7 +440,8 @@ struct DiffOut {  // what two maps become one output row with
   float post, eps;
 };
 
-template <typename T, int MAPS>
+// MC: value columns per lane, dv <= 16 MC
+template <typename T, int MAPS, int MC>
 __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
                                                         float* __restrict__ part_ml, const float* __restrict__ q,
                                                         const T* __restrict__ k_cache, const T* __restrict__ v_cache,
@@ -477,11 +478,11 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
   const int k_begin = blockIdx.z * per, k_end = min(n_vis, k_begin + per);
   for (int i = l; i < dk; i += 16) sq[r * qs + i] = q[((size_t)tok * H + head) * dk + i];
   const int* trow = table + (size_t)req_rows[b] * table_stride;
-  float o[MAPS][kSinkMaxC], m[MAPS], lsum[MAPS];
+  float o[MAPS][MC], m[MAPS], lsum[MAPS];
 #pragma unroll
   for (int a = 0; a < MAPS; ++a) {
 #pragma unroll
-    for (int i = 0; i < kSinkMaxC; ++i) o[a][i] = 0.f;
+    for (int i = 0; i < MC; ++i) o[a][i] = 0.f;
     m[a] = -INFINITY;
     lsum[a] = 0.f;
   }
@@ -537,7 +538,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
 #pragma unroll
     for (int a = 0; a < MAPS; ++a)
 #pragma unroll
-      for (int i = 0; i < kSinkMaxC; ++i) {
+      for (int i = 0; i < MC; ++i) {
         const int c = l + 16 * i;
         if (c < dv) {
           float acc = o[a][i] * alpha[a];
@@ -550,7 +551,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
     const float f0 = 1.0f / lsum[0], f1 = df.lam[0] / lsum[MAPS - 1];  // a row that is not valid holds no sum and is not written
     float ss = 0.f;
 #pragma unroll
-    for (int i = 0; i < kSinkMaxC; ++i) {
+    for (int i = 0; i < MC; ++i) {
       o[0][i] = o[0][i] * f0 - o[MAPS - 1][i] * f1;
       if (l + 16 * i < dv) ss = fmaf(o[0][i], o[0][i], ss);
     }
@@ -560,7 +561,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
     const float f = df.post / sqrtf(ss / (float)dv + df.eps);
     const T* gate = cp<T>(df.gate);
 #pragma unroll
-    for (int i = 0; i < kSinkMaxC; ++i) {
+    for (int i = 0; i < MC; ++i) {
       const int c = l + 16 * i;
       if (c < dv) {
         const float gz = gate ? sigmoidf_(ld(gate + (size_t)tok * df.ld_gate + (size_t)head * dv + c)) : 1.f;
@@ -576,7 +577,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
     const float em = expf(m[0] - mf);
     const float f = em / (lsum[0] * em + (sink ? expf(sk_h - mf) : 0.f));
 #pragma unroll
-    for (int i = 0; i < kSinkMaxC; ++i) {
+    for (int i = 0; i < MC; ++i) {
       const int c = l + 16 * i;
       if (c < dv) st(out + (size_t)tok * ld_out + (size_t)head * dv + c, o[0][i] * f);
     }
@@ -586,7 +587,7 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
   for (int a = 0; a < MAPS; ++a) {
     const size_t row = (((size_t)blockIdx.z * total_q + tok) * H + head) * MAPS + a;
 #pragma unroll
-    for (int i = 0; i < kSinkMaxC; ++i) {
+    for (int i = 0; i < MC; ++i) {
       const int c = l + 16 * i;
       if (c < dv) part_o[row * dv + c] = o[a][i];
     }
@@ -871,9 +872,9 @@ __global__ __launch_bounds__(64) void diff_merge_kernel(T* __restrict__ out, int
     }
     f[a] = (a == 0 ? 1.0f : -df.lam[0]) / den;
   }
-  float o[4], ss = 0.f;  // dv <= 256
+  float o[kSinkMaxDv / 64], ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < kSinkMaxDv / 64; ++i) {
     const int c = threadIdx.x + 64 * i;
     o[i] = 0.f;
     if (c < dv) {
@@ -889,7 +890,7 @@ __global__ __launch_bounds__(64) void diff_merge_kernel(T* __restrict__ out, int
   const float n = df.post / sqrtf(wave_sum(ss) / (float)dv + df.eps);
   const T* gate = cp<T>(df.gate);
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < kSinkMaxDv / 64; ++i) {
     const int c = threadIdx.x + 64 * i;
     if (c < dv) {
       const float gz = gate ? sigmoidf_(ld(gate + t * df.ld_gate + (size_t)h * dv + c)) : 1.f;
@@ -1139,7 +1140,7 @@ int sink_attn_any(void* out, int64_t ld_out, const float* q, const void* k_cache
                   const int* req_rows, const int* seq_lens, const int* cu_q, int batch, int total_q, int H, int G, int d, int dv, float scale,
                   int window, int keep, const float* sink, DiffOut df, int dtype, int splits, float* workspace, hipStream_t s) {
   MIX_REQUIRE(out && q && k_cache && v_cache && table && req_rows && seq_lens && cu_q && dtype_ok(dtype), "sink_attn: null pointer / dtype");
-  MIX_REQUIRE(batch >= 1 && total_q >= 0 && H >= 1 && G >= 1 && H % G == 0 && d >= 1 && dv >= 1 && dv <= 16 * kSinkMaxC && keep >= 0 &&
+  MIX_REQUIRE(batch >= 1 && total_q >= 0 && H >= 1 && G >= 1 && H % G == 0 && d >= 1 && dv >= 1 && dv <= kSinkMaxDv && keep >= 0 &&
                   ld_out >= (int64_t)H * dv,
               "sink_attn: bad sizes H %d G %d d %d dv %d", H, G, d, dv);
   MIX_REQUIRE(splits >= 1 && splits <= 1024 && (splits == 1 || workspace), "sink_attn: %d splits need a workspace", splits);
@@ -1187,12 +1188,18 @@ int sink_attn_any(void* out, int64_t ld_out, const float* q, const void* k_cache
   MIX_REQUIRE(lds <= 160 * 1024, "sink_attn: heads of %d / %d do not fit LDS", d, dv);
   const int groups = (total_q + QT - 1) / QT + batch;  // every request may end with one partial group
   MIX_REQUIRE((int64_t)G * hblocks <= 65535, "sink_attn: too many heads");
-  DISPATCH_T(dtype, MIX_REQUIRE((ensure_lds((const void*)sink_attn_kernel<T, MAPS>, lds) == 0), "sink_attn: LDS request refused");
-             hipLaunchKernelGGL((sink_attn_kernel<T, MAPS>), dim3(groups, G * hblocks, splits), dim3(256), lds, s, mp<T>(out), ld_out, part_o,
-                                part_ml, q, cp<T>(k_cache), cp<T>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H,
-                                G, d, dv, scale, window, keep, sink, df, QT, HB, KT, splits);
-             MIX_LAUNCHED("sink_attn");
+#define SINK_PLAIN(MC)                                                                                                                       \
+  DISPATCH_T(dtype, MIX_REQUIRE((ensure_lds((const void*)sink_attn_kernel<T, MAPS, MC>, lds) == 0), "sink_attn: LDS request refused");         \
+             hipLaunchKernelGGL((sink_attn_kernel<T, MAPS, MC>), dim3(groups, G * hblocks, splits), dim3(256), lds, s, mp<T>(out), ld_out, part_o, \
+                                part_ml, q, cp<T>(k_cache), cp<T>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H,  \
+                                G, d, dv, scale, window, keep, sink, df, QT, HB, KT, splits);                                                 \
+             MIX_LAUNCHED("sink_attn");                                                                                                       \
              return (sink_merge_launch<T, MAPS>(s, mp<T>(out), ld_out, part_o, part_ml, total_q, H, dv, splits, sink, df));)
+  if (dv <= 256) {
+    SINK_PLAIN(16)
+  }
+  SINK_PLAIN(64)
+#undef SINK_PLAIN
 }
 
 }  // namespace

@@ -138,14 +138,22 @@ __device__ __forceinline__ Q4 load8(const float* p, int n, bool vec) {
             bf16_bits(f[4]) | (bf16_bits(f[5]) << 16), bf16_bits(f[6]) | (bf16_bits(f[7]) << 16)};
 }
 
+// two fp32 numbers as packed bf16 (round to nearest even), one instruction
+typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
+typedef float f32x2_t __attribute__((ext_vector_type(2)));
+__device__ __forceinline__ uint32_t pack_bf16(float a, float b) {
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2_t{a, b}, bf16x2_t));
+}
+
 typedef __attribute__((ext_vector_type(4))) short s16x4_t;
 typedef __attribute__((address_space(3))) s16x4_t lds_s16x4_t;
 
-// Which request and which of its QT-token groups workgroup `blockIdx.x` owns: group counts ceil(new tokens / QT) of up to 256
+// Which request and which of its QT-token groups the workgroup with this index (default: blockIdx.x) owns: group counts ceil(new tokens / QT) of up to 256
 // requests at a time, scanned by the whole workgroup (one pass of independent loads instead of one thread walking the batch).
 // Leaves request -1 for workgroups past the last group.  cnt: 256 ints of LDS; every thread of the (256-thread) workgroup calls.
-__device__ __forceinline__ void find_group(const int* __restrict__ cu_q, int B, int QT, int* cnt, int* s_req, int* s_tok0) {
+__device__ __forceinline__ void find_group(const int* __restrict__ cu_q, int B, int QT, int* cnt, int* s_req, int* s_tok0, int index = -1) {
   const int tid = threadIdx.x;
+  if (index < 0) index = (int)blockIdx.x;
   if (tid == 0) *s_req = -1;
   int base = 0;
   for (int c0 = 0; c0 < B; c0 += 256) {
@@ -160,7 +168,7 @@ __device__ __forceinline__ void find_group(const int* __restrict__ cu_q, int B, 
       __syncthreads();
     }
     const int incl = cnt[tid], total = cnt[255];
-    const int target = (int)blockIdx.x - base;
+    const int target = index - base;
     if (b < B && target >= incl - g && target < incl) {
       *s_req = b;
       *s_tok0 = (target - (incl - g)) * QT;

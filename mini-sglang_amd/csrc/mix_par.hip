@@ -279,6 +279,107 @@ __global__ __launch_bounds__(256) void qk_prep_kernel(const T* __restrict__ proj
   for (int e = threadIdx.x; e < Gv * dv; e += 256) st(v_cache + slot * Gv * dv + e, ld(src + vo + e) + (bias ? bias[vo + e] : 0.f));
 }
 
+// The same with 16-byte accesses and every head in the registers of `lph` neighbouring lanes (a power of two, 8 entries each; value heads:
+// lphv), for head sizes that are multiples of 8 and rotations whose pairs keep 8-entry pieces together: a piece's partners lie in the piece
+// itself (interleaved) or are another lane's piece.
+__device__ __forceinline__ float group_sum(float v, int width) {
+  for (int o = width >> 1; o >= 1; o >>= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void qk_prep_vec_kernel(const T* __restrict__ proj, int64_t ld_proj, const float* __restrict__ bias,
+                                                          float* __restrict__ q_out, T* __restrict__ k_cache, T* __restrict__ v_cache,
+                                                          const int* __restrict__ out_loc, const int* __restrict__ positions,
+                                                          const float* __restrict__ cos_sin, int rd, int interleaved, int unit, float eps,
+                                                          const T* __restrict__ q_w, const T* __restrict__ k_w, int H, int G, int Gv, int d,
+                                                          int dv, int lph, int lphv) {
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const T* src = proj + (size_t)t * ld_proj;
+  const size_t slot = (size_t)out_loc[t];
+  const float* cs = cos_sin ? cos_sin + (size_t)positions[t] * rd : nullptr;
+  const int half = rd >> 1;
+  auto read = [&](size_t at, float (&v)[8]) {
+    read8(src + at, v);
+    if (bias) {
+      float b[8];
+      read8(bias + at, b);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] += b[e];
+    }
+  };
+  auto to_unit = [&](float (&v)[8], int width, int n) {  // pieces past the head's end hold zeros
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss = fmaf(v[e], v[e], ss);
+    const float f = 1.0f / sqrtf(group_sum(ss, width) / (float)n + eps);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] *= f;
+  };
+  const int sub = tid & (lph - 1), c0 = sub * 8;
+  for (int h0 = 0; h0 < H + G; h0 += 256 / lph) {  // every lane stays in the loop: heads exchange pieces
+    const int hh = h0 + tid / lph;
+    const bool live = hh < H + G && c0 < d;
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (live) read((size_t)hh * d + c0, v);
+    if (q_w) {
+      to_unit(v, lph, d);
+      if (live) {
+        float w[8];
+        read8((hh < H ? q_w : k_w) + c0, w);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] *= w[e];
+      }
+    }
+    if (rd > 0) {
+      if (interleaved) {
+        if (c0 < rd) {
+          const float4 c = *reinterpret_cast<const float4*>(cs + (c0 >> 1)), n = *reinterpret_cast<const float4*>(cs + half + (c0 >> 1));
+          const float cv[4] = {c.x, c.y, c.z, c.w}, sv[4] = {n.x, n.y, n.z, n.w};
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const float a = v[2 * i], b = v[2 * i + 1];
+            v[2 * i] = a * cv[i] - b * sv[i];
+            v[2 * i + 1] = b * cv[i] + a * sv[i];
+          }
+        }
+      } else {
+        const bool lower = c0 < half;
+        const int other = c0 < rd ? (lower ? sub + (half >> 3) : sub - (half >> 3)) : sub;
+        const int lane = (tid & 63 & ~(lph - 1)) + other;
+        float o[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = __shfl(v[e], lane, 64);
+        if (c0 < rd) {
+          const int i = lower ? c0 : c0 - half;
+          float c[8], n[8];
+          read8(cs + i, c);
+          read8(cs + half + i, n);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) v[e] = lower ? v[e] * c[e] - o[e] * n[e] : v[e] * c[e] + o[e] * n[e];
+        }
+      }
+    }
+    if (unit & 1) to_unit(v, lph, d);
+    if (live) {
+      if (hh < H)
+        write8(q_out + ((size_t)t * H + hh) * d + c0, v);
+      else
+        write8(k_cache + (slot * G + hh - H) * d + c0, v);
+    }
+  }
+  const size_t vo = (size_t)(H + G) * d;
+  const int cv = (tid & (lphv - 1)) * 8;
+  for (int g0 = 0; g0 < Gv; g0 += 256 / lphv) {
+    const int g = g0 + tid / lphv;
+    const bool live = g < Gv && cv < dv;
+    float v[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (live) read(vo + (size_t)g * dv + cv, v);
+    if (unit & 2) to_unit(v, lphv, dv);
+    if (live) write8(v_cache + (slot * Gv + g) * dv + cv, v);
+  }
+}
+
 // ------------------------------------------------------------------------------------------------ sigmoid attention
 // A workgroup = 16 query rows (QT tokens of one request x HB query heads of ONE key/value head) x 16 lanes, one range of the keys.
 // Keys and values of the tile go through LDS as fp32; weight of a visible key = sigmoid(cap * tanh(scale q.k / cap) + pb[h])
@@ -794,6 +895,19 @@ int msgl_mix_qk_prep(const void* proj, int64_t ld_proj, const float* bias, float
   if (tokens == 0) return MSGL_MIX_OK;
   const size_t lds = (size_t)(H + G) * d * sizeof(float) * (q_w ? 2 : 1);
   hipStream_t s = static_cast<hipStream_t>(stream);
+  bool vec = d % 8 == 0 && dv % 8 == 0 && d <= 512 && dv <= 512 && ld_proj % 8 == 0 && rot_dims % (interleaved ? 8 : 16) == 0;
+  for (const void* p : {proj, (const void*)bias, (const void*)q_out, (const void*)k_cache, (const void*)v_cache, (const void*)cos_sin, q_w, k_w})
+    vec = vec && ((uintptr_t)p & 15u) == 0;
+  if (vec) {
+    int lph = 1, lphv = 1;
+    while (lph * 8 < d) lph <<= 1;
+    while (lphv * 8 < dv) lphv <<= 1;
+    DISPATCH_T(dtype, hipLaunchKernelGGL(qk_prep_vec_kernel<T>, dim3(tokens), dim3(256), 0, s, cp<T>(proj), ld_proj, bias, q_out, mp<T>(k_cache),
+                                         mp<T>(v_cache), out_loc, positions, cos_sin, rot_dims, interleaved, unit, eps, cp<T>(q_w), cp<T>(k_w),
+                                         H, G, Gv, d, dv, lph, lphv);)
+    MIX_LAUNCHED("qk_prep");
+    return MSGL_MIX_OK;
+  }
   DISPATCH_T(dtype, MIX_REQUIRE(ensure_lds((const void*)qk_prep_kernel<T>, lds) == 0, "qk_prep: heads do not fit LDS");
              hipLaunchKernelGGL(qk_prep_kernel<T>, dim3(tokens), dim3(256), lds, s, cp<T>(proj), ld_proj, bias, q_out, mp<T>(k_cache),
                                 mp<T>(v_cache), out_loc, positions, cos_sin, rot_dims, interleaved, unit, eps, cp<T>(q_w), cp<T>(k_w), H, G,

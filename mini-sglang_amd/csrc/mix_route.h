@@ -169,16 +169,16 @@ __device__ __forceinline__ void select_experts_wave(float* s, float* c, float* g
   for (int k = lane; k < top; k += 64) wts[k] = gs[G + k] * inv;
 }
 
-// Router logits of ONE row by a 256-thread workgroup: sc[e] = router[e] . row (row: W fp32 numbers in LDS, as the router reads them; the
-// caller has synchronized after writing it and synchronizes before reading sc).  A wave takes experts wave, wave + 4, ...; up to kRouteAcc
+// Router logits of ONE row by a workgroup of WAVES waves: sc[e] = router[e] . row (row: W fp32 numbers in LDS, as the router reads them; the
+// caller has synchronized after writing it and synchronizes before reading sc).  A wave takes experts wave, wave + WAVES, ...; up to kRouteAcc
 // of them at once, so that one pass over the row has that many independent weight loads in flight per lane (element order per expert:
 // lane-strided, then the wave reduction: fixed).
-template <typename T>
-__device__ __forceinline__ void router_logits256(const float* row, const T* __restrict__ router, int E, int W, float* sc) {
+template <int WAVES, typename T>
+__device__ __forceinline__ void router_logits(const float* row, const T* __restrict__ router, int E, int W, float* sc) {
   constexpr int kRouteAcc = 8;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const bool wide = (W & 7) == 0 && ((uintptr_t)router & 15u) == 0;
-  for (int e0 = wave; e0 < E; e0 += 4 * kRouteAcc) {
+  for (int e0 = wave; e0 < E; e0 += WAVES * kRouteAcc) {
     float acc[kRouteAcc];
 #pragma unroll
     for (int a = 0; a < kRouteAcc; ++a) acc[a] = 0.f;
@@ -189,7 +189,7 @@ __device__ __forceinline__ void router_logits256(const float* row, const T* __re
         for (int u = 0; u < 8; ++u) hv[u] = row[i + u];
 #pragma unroll
         for (int a = 0; a < kRouteAcc; ++a) {
-          const int e = e0 + 4 * a;
+          const int e = e0 + WAVES * a;
           if (e < E) {
             float wv[8];
             read8(router + (size_t)e * W + i, wv);
@@ -203,14 +203,14 @@ __device__ __forceinline__ void router_logits256(const float* row, const T* __re
         const float hv = row[i];
 #pragma unroll
         for (int a = 0; a < kRouteAcc; ++a) {
-          const int e = e0 + 4 * a;
+          const int e = e0 + WAVES * a;
           if (e < E) acc[a] = fmaf(hv, ld(router + (size_t)e * W + i), acc[a]);
         }
       }
     }
 #pragma unroll
     for (int a = 0; a < kRouteAcc; ++a) {
-      const int e = e0 + 4 * a;
+      const int e = e0 + WAVES * a;
       const float v = wave_sum(acc[a]);
       if (e < E && lane == 0) sc[e] = v;
     }

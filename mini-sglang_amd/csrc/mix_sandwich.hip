@@ -76,18 +76,29 @@ __device__ __forceinline__ void norm_row(float (&v)[NCH][8], const T* __restrict
   }
 }
 
+// TPR threads per row: 64 (a wave), 256, or, for a routed row, 1024 (the row itself needs W / 8 of them, its router all)
 template <typename T, int NCH, int TPR, bool ROUTE>
-__global__ __launch_bounds__(256) void join_norm_vec_kernel(JoinArgs a) {
-  static_assert(!ROUTE || TPR == 256, "a routed row has a workgroup of its own");
-  extern __shared__ float lds[];  // 4 floats; with ROUTE W + 2 E + G + top more
+__global__ __launch_bounds__(TPR == 64 ? 256 : TPR) void join_norm_vec_kernel(JoinArgs a) {
+  static_assert(!ROUTE || TPR == 1024, "a routed row has a large workgroup of its own");
+  extern __shared__ float lds[];  // 16 floats; with ROUTE W + 2 E + G + top more
   const int lane = TPR == 64 ? threadIdx.x & 63 : threadIdx.x;
   const int t = TPR == 64 ? blockIdx.x * 4 + (threadIdx.x >> 6) : blockIdx.x;
-  if (t >= a.rows) return;  // whole waves, and no barrier below, when TPR = 64; never when TPR = 256
+  if (t >= a.rows) return;  // whole waves, and no barrier below, when TPR = 64; never otherwise
   auto reduce = [&](float v) {
     if constexpr (TPR == 64)
       return wave_sum(v);
-    else
+    else if constexpr (TPR == 256)
       return block_sum256(v, lds);
+    else {
+      v = wave_sum(v);
+      __syncthreads();
+      if ((threadIdx.x & 63) == 0) lds[threadIdx.x >> 6] = v;
+      __syncthreads();
+      float s = 0.f;
+#pragma unroll
+      for (int w = 0; w < TPR / 64; ++w) s += lds[w];
+      return s;
+    }
   };
   const int W = a.W, nch = W >> 3;
   float x[NCH][8];
@@ -163,7 +174,7 @@ __global__ __launch_bounds__(256) void join_norm_vec_kernel(JoinArgs a) {
     if (ch < nch) write8(mp<T>(a.h_out) + (size_t)t * W + ch * 8, x[j]);
   }
   if constexpr (ROUTE) {
-    float* row = lds + 4;
+    float* row = lds + 16;
     float* sc = row + W;
 #pragma unroll
     for (int j = 0; j < NCH; ++j) {
@@ -178,7 +189,7 @@ __global__ __launch_bounds__(256) void join_norm_vec_kernel(JoinArgs a) {
       }
     }
     __syncthreads();
-    router_logits256(row, cp<T>(a.router), a.E, W, sc);
+    router_logits<TPR / 64>(row, cp<T>(a.router), a.E, W, sc);
     __syncthreads();
     if (threadIdx.x < 64)
       select_experts_wave<T>(sc, sc + a.E, sc + 2 * a.E, cp<T>(a.bias), a.E, a.top, a.G, a.keep, a.rule, a.pick + (size_t)t * a.top,
@@ -232,7 +243,7 @@ __global__ __launch_bounds__(256) void join_norm_kernel(JoinArgs a) {
   }
   if (!a.router) return;
   __syncthreads();
-  router_logits256(x, cp<T>(a.router), a.E, W, s);
+  router_logits<4>(x, cp<T>(a.router), a.E, W, s);
   __syncthreads();
   if (threadIdx.x < 64)
     select_experts_wave<T>(s, s + a.E, s + 2 * a.E, cp<T>(a.bias), a.E, a.top, a.G, a.keep, a.rule, a.pick + (size_t)t * a.top,
@@ -288,17 +299,10 @@ __global__ __launch_bounds__(256) void gate_mul_kernel(T* __restrict__ out, cons
 
 bool aligned16(const void* p) { return ((uintptr_t)p & 15u) == 0; }
 
-template <typename T, int NCH, int TPR>
+template <typename T, int NCH, int TPR, bool ROUTE = false>
 int join_launch(const JoinArgs& a, size_t lds, hipStream_t s) {
-  if constexpr (TPR == 256) {
-    if (a.router) {
-      MIX_REQUIRE(ensure_lds((const void*)join_norm_vec_kernel<T, NCH, TPR, true>, lds) == 0, "join_norm: row of %d does not fit LDS", a.W);
-      hipLaunchKernelGGL((join_norm_vec_kernel<T, NCH, TPR, true>), dim3(a.rows), dim3(256), lds, s, a);
-      MIX_LAUNCHED("join_norm (routed)");
-      return MSGL_MIX_OK;
-    }
-  }
-  hipLaunchKernelGGL((join_norm_vec_kernel<T, NCH, TPR, false>), dim3(TPR == 64 ? (a.rows + 3) / 4 : a.rows), dim3(256), 4 * sizeof(float), s, a);
+  MIX_REQUIRE(ensure_lds((const void*)join_norm_vec_kernel<T, NCH, TPR, ROUTE>, lds) == 0, "join_norm: row of %d does not fit LDS", a.W);
+  hipLaunchKernelGGL((join_norm_vec_kernel<T, NCH, TPR, ROUTE>), dim3(TPR == 64 ? (a.rows + 3) / 4 : a.rows), dim3(TPR == 64 ? 256 : TPR), lds, s, a);
   MIX_LAUNCHED("join_norm");
   return MSGL_MIX_OK;
 }
@@ -312,13 +316,11 @@ int join_pick(const JoinArgs& a, hipStream_t s) {
                         (const void*)a.h_out})
     vec = vec && aligned16(p);
   if (vec) {
-    const size_t lds = (4 + (a.router ? W + route : 0)) * sizeof(float);
-    // many rows: a wave owns a row and nothing meets at a barrier; few rows: a workgroup owns one, for four times the loads in flight
-    if (!a.router && a.rows >= 1024) {
-      if (W <= 512) return join_launch<T, 1, 64>(a, lds, s);
-      if (W <= 1024) return join_launch<T, 2, 64>(a, lds, s);
-      if (W <= 2048) return join_launch<T, 4, 64>(a, lds, s);
-    }
+    const size_t lds = (16 + (a.router ? W + route : 0)) * sizeof(float);
+    if (a.router) return join_launch<T, 1, 1024, true>(a, lds, s);
+    // many short rows: a wave owns a row and nothing meets at a barrier; otherwise a workgroup owns one, for more loads in flight per row
+    if (a.rows >= 1024 && W <= 512) return join_launch<T, 1, 64>(a, lds, s);
+    if (a.rows >= 1024 && W <= 1024) return join_launch<T, 2, 64>(a, lds, s);
     if (W <= 2048) return join_launch<T, 1, 256>(a, lds, s);
     if (W <= 4096) return join_launch<T, 2, 256>(a, lds, s);
     return join_launch<T, 4, 256>(a, lds, s);

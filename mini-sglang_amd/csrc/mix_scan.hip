@@ -604,11 +604,16 @@ __global__ __launch_bounds__(256) void sink_attn_kernel(T* __restrict__ out, int
 //   S^T[16 keys x 16 rows] = K . Q^T     per 16-key subtile KC x v_mfma_f32_16x16x32_bf16 (Q fragments in registers, rounded to bf16 once)
 //   ONE fp32 softmax step for the tile in the lane that holds the scores (a query row's 16 keys; the row's other keys sit in the
 //   lanes 16, 32 and 48 further on): new maximum, rescale of the row's sum and output, weights as bf16 B operands;
-//   O^T[16 v x 16 rows] += V^T . P^T     VC x v_mfma_f32_16x16x16_bf16, V^T fragments read TRANSPOSED out of the row-major value
-//   tile (ds_read_b64_tr_b16).
+//   O^T[16 v x 16 rows] += V^T . P^T     VC x v_mfma_f32_16x16x32_bf16 per 32 keys, V^T fragments read TRANSPOSED out of the row-major
+//   value tile (ds_read_b64_tr_b16).  The order of a product's 32 summands is free: lane group g takes keys 4 g .. 4 g + 3 of two
+//   neighbouring subtiles on both sides, which is how the scores lie in their lanes.
+// The scale and log2(e) enter with Q, so that a weight is one subtraction and one exp2; a tile that every row of the workgroup sees
+// whole is not masked; a wave rescales its output only when a maximum of its rows has moved.
+// SPREAD (steps with at most 16 query rows per workgroup, decode): the 16 rows belong to all four waves, wave w takes the w-th 16 keys of
+// every tile with a softmax state of its own, and the four states are joined through LDS at the end.
 constexpr int kNKT = 64;
 
-template <int KC, int VC, int MAPS>
+template <int KC, int VC, int MAPS, bool SPREAD>
 __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void sink_attn_mfma_kernel(bf16_t* __restrict__ out, int64_t ld_out, float* __restrict__ part_o,
                                                              float* __restrict__ part_ml, const float* __restrict__ q,
                                                              const bf16_t* __restrict__ k_cache, const bf16_t* __restrict__ v_cache,
@@ -623,7 +628,7 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
   uint16_t* sv = smem + kNKT * KS;   // [kNKT][VS]
   __shared__ int s_req, s_tok0, s_cnt[256];
   __shared__ int s_slot[2][kNKT];
-  find_group(cu_q, B, QT, s_cnt, &s_req, &s_tok0);
+  find_group(cu_q, B, QT, s_cnt, &s_req, &s_tok0, (int)(gridDim.x - 1 - blockIdx.x));  // last tokens, with the most keys, first
   const int b = s_req;
   if (b < 0) return;
   const int rep = H / G, hblocks = (rep + HB - 1) / HB;
@@ -632,7 +637,7 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
   const int start = seq_lens[b] - q_len;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int lr = lane & 15, lg = lane >> 4;
-  const int r = wave * 16 + lr;
+  const int r = SPREAD ? lr : wave * 16 + lr;
   const int tl = s_tok0 + r / HB, hh = h0 + r % HB;
   const bool valid = r < QT * HB && tl < q_len && hh < (kvh + 1) * rep;
   const int tok = cu_q[b] + (valid ? tl : s_tok0);
@@ -647,6 +652,9 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
   const int k_begin = z * per, k_end = min(n_vis, k_begin + per);
   auto key_at = [&](int v) { return v < keep_eff ? v : v + shift; };
   const bool wave_live = __builtin_amdgcn_ballot_w64(valid) != 0;
+  const float scale2 = scale * 1.4426950408889634f;
+  // keys up to here are seen by every row of the workgroup, and from here on the window's lower edge too
+  const int all_hi = start + s_tok0, all_lo = window > 0 ? max(0, start + last_tok - window + 1) : 0;
   bf16x8_t qf[MAPS][KC];
   f32x4_t o[MAPS][VC];
   float m[MAPS], lsum[MAPS];  // the row's maximum (the same in its four lanes) and this lane's share of the row's sum
@@ -656,8 +664,10 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
 #pragma unroll
     for (int kc = 0; kc < KC; ++kc) {
       const int k = kc * 32 + lg * 8;
-      Q4 v = (valid && k < d) ? load8(qrow + k, d - k, (d & 3) == 0) : Q4{0u, 0u, 0u, 0u};
-      qf[a][kc] = __builtin_bit_cast(bf16x8_t, v);
+      float f[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[e] = valid && k + e < d ? qrow[k + e] * scale2 : 0.f;
+      qf[a][kc] = __builtin_bit_cast(bf16x8_t, Q4{pack_bf16(f[0], f[1]), pack_bf16(f[2], f[3]), pack_bf16(f[4], f[5]), pack_bf16(f[6], f[7])});
     }
 #pragma unroll
     for (int vt = 0; vt < VC; ++vt) o[a][vt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -709,8 +719,10 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
     __syncthreads();
     if (j0 + kNKT < k_end) request(j0 + kNKT, buf ^ 1);
     if (!wave_live) continue;
-    constexpr int NKS = kNKT / 16;
-    s16x4_t pf[MAPS][NKS];
+    constexpr int NKS = SPREAD ? 1 : kNKT / 16;
+    const int ks0 = SPREAD ? wave : 0;
+    const bool whole = j0 + kNKT <= k_end && key_at(j0 + kNKT - 1) <= all_hi && key_at(j0) >= all_lo;
+    uint2 pf[MAPS][NKS];
 #pragma unroll
     for (int a = 0; a < MAPS; ++a) {
       f32x4_t sc[NKS];
@@ -720,50 +732,68 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
         f32x4_t sacc{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kc = 0; kc < KC; ++kc) {
-          const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&sk[(ks * 16 + lr) * KS + a * KM + kc * 32 + lg * 8]);
+          const bf16x8_t kf = *reinterpret_cast<const bf16x8_t*>(&sk[((ks0 + ks) * 16 + lr) * KS + a * KM + kc * 32 + lg * 8]);
           sacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[a][kc], sacc, 0, 0, 0);
         }
+        if (!whole) {
 #pragma unroll
-        for (int c = 0; c < 4; ++c) {
-          const int v = j0 + ks * 16 + 4 * lg + c, j = key_at(v);
-          const float s = (j <= limit && (j >= lo_row || j < keep) && v < k_end) ? sacc[c] * scale : -INFINITY;
-          sacc[c] = s;
-          tmax = fmaxf(tmax, s);
+          for (int c = 0; c < 4; ++c) {
+            const int v = j0 + (ks0 + ks) * 16 + 4 * lg + c, j = key_at(v);
+            if (!(j <= limit && (j >= lo_row || j < keep) && v < k_end)) sacc[c] = -INFINITY;
+          }
         }
+        tmax = fmaxf(tmax, fmaxf(fmaxf(sacc[0], sacc[1]), fmaxf(sacc[2], sacc[3])));
         sc[ks] = sacc;
       }
       tmax = fmaxf(tmax, __shfl_xor(tmax, 16, 64));
       tmax = fmaxf(tmax, __shfl_xor(tmax, 32, 64));
       const float m_new = fmaxf(m[a], tmax);
-      const float alpha = m_new == -INFINITY ? 1.0f : __expf(m[a] - m_new);
+      const float base = m_new == -INFINITY ? 0.f : m_new;  // no visible key yet: every weight below is exp2(-inf) = 0
+      const float alpha = __builtin_amdgcn_exp2f(m[a] - base);
       float psum = 0.f;
 #pragma unroll
       for (int ks = 0; ks < NKS; ++ks) {
         float pe[4];
 #pragma unroll
         for (int c = 0; c < 4; ++c) {
-          pe[c] = sc[ks][c] == -INFINITY ? 0.f : __expf(sc[ks][c] - m_new);
+          pe[c] = __builtin_amdgcn_exp2f(sc[ks][c] - base);
           psum += pe[c];
         }
-        const uint32_t p01 = bf16_bits(pe[0]) | (bf16_bits(pe[1]) << 16), p23 = bf16_bits(pe[2]) | (bf16_bits(pe[3]) << 16);
-        pf[a][ks] = __builtin_bit_cast(s16x4_t, uint2{p01, p23});
+        pf[a][ks] = uint2{pack_bf16(pe[0], pe[1]), pack_bf16(pe[2], pe[3])};
       }
       lsum[a] = fmaf(lsum[a], alpha, psum);
+      if (__builtin_amdgcn_ballot_w64(m_new > m[a]) != 0) {
+#pragma unroll
+        for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) o[a][vt][c] *= alpha;
+      }
       m[a] = m_new;
-#pragma unroll
-      for (int vt = 0; vt < VC; ++vt)
-#pragma unroll
-        for (int c = 0; c < 4; ++c) o[a][vt][c] *= alpha;
     }
-#pragma unroll
-    for (int ks = 0; ks < NKS; ++ks) {
-      if (j0 + ks * 16 >= k_end) break;
-      const uint16_t* vbase = &sv[(ks * 16 + 4 * lg + (lr >> 2)) * VS + 4 * (lr & 3)];
+    const uint16_t* vbase = &sv[(ks0 * 16 + 4 * lg + (lr >> 2)) * VS + 4 * (lr & 3)];
+    if constexpr (SPREAD) {
 #pragma unroll
       for (int vt = 0; vt < VC; ++vt) {
         const s16x4_t vf = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)(vbase + vt * 16));
 #pragma unroll
-        for (int a = 0; a < MAPS; ++a) o[a][vt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, pf[a][ks], o[a][vt], 0, 0, 0);
+        for (int a = 0; a < MAPS; ++a)
+          o[a][vt] = __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(vf, __builtin_bit_cast(s16x4_t, pf[a][0]), o[a][vt], 0, 0, 0);
+      }
+    } else {
+#pragma unroll
+      for (int kp = 0; kp < NKS / 2; ++kp) {
+        if (j0 + kp * 32 >= k_end) break;
+#pragma unroll
+        for (int vt = 0; vt < VC; ++vt) {
+          const s16x4_t v0 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)(vbase + kp * 32 * VS + vt * 16));
+          const s16x4_t v1 = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4_t*)(vbase + (kp * 32 + 16) * VS + vt * 16));
+          const bf16x8_t vf = __builtin_bit_cast(bf16x8_t, __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+          for (int a = 0; a < MAPS; ++a) {
+            const Q4 pq{pf[a][2 * kp].x, pf[a][2 * kp].y, pf[a][2 * kp + 1].x, pf[a][2 * kp + 1].y};
+            o[a][vt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, __builtin_bit_cast(bf16x8_t, pq), o[a][vt], 0, 0, 0);
+          }
+        }
       }
     }
   }
@@ -772,6 +802,62 @@ __global__ __launch_bounds__(256, MAPS == 2 && KC <= 2 && VC <= 8 ? 2 : 1) void 
     lsum[a] += __shfl_xor(lsum[a], 16, 64);
     lsum[a] += __shfl_xor(lsum[a], 32, 64);
   }
+  if constexpr (SPREAD) {
+    // join the four waves' states: factors from their maxima, then the outputs pairwise (waves 2, 3 onto 0, 1, then 1 onto 0)
+    static_assert((size_t)2 * MAPS * VC * 4 * 64 * sizeof(float) <= (size_t)kNKT * (KS + VS) * sizeof(uint16_t), "two waves' outputs fit the tiles' LDS");
+    __shared__ float s_ml[4][MAPS][2][16];
+    float* so = reinterpret_cast<float*>(smem) + lane;
+    if (lg == 0) {
+#pragma unroll
+      for (int a = 0; a < MAPS; ++a) {
+        s_ml[wave][a][0][lr] = m[a];
+        s_ml[wave][a][1][lr] = lsum[a];
+      }
+    }
+    __syncthreads();  // also: every wave has read its last tile
+#pragma unroll
+    for (int a = 0; a < MAPS; ++a) {
+      float M = -INFINITY, L = 0.f;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) M = fmaxf(M, s_ml[w][a][0][lr]);
+      const float base = M == -INFINITY ? 0.f : M;
+#pragma unroll
+      for (int w = 0; w < 4; ++w) L = fmaf(s_ml[w][a][1][lr], __builtin_amdgcn_exp2f(s_ml[w][a][0][lr] - base), L);
+      const float f = __builtin_amdgcn_exp2f(m[a] - base);
+#pragma unroll
+      for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+        for (int c = 0; c < 4; ++c) o[a][vt][c] *= f;
+      m[a] = M;
+      lsum[a] = L;
+    }
+    auto at = [&](int part, int a, int vt, int c) { return (((part * MAPS + a) * VC + vt) * 4 + c) * 64; };
+#pragma unroll
+    for (int half = 2; half >= 1; half >>= 1) {
+      if (wave >= half && wave < 2 * half) {
+#pragma unroll
+        for (int a = 0; a < MAPS; ++a)
+#pragma unroll
+          for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+            for (int c = 0; c < 4; ++c) so[at(wave - half, a, vt, c)] = o[a][vt][c];
+      }
+      __syncthreads();
+      if (wave < half) {
+#pragma unroll
+        for (int a = 0; a < MAPS; ++a)
+#pragma unroll
+          for (int vt = 0; vt < VC; ++vt)
+#pragma unroll
+            for (int c = 0; c < 4; ++c) o[a][vt][c] += so[at(wave, a, vt, c)];
+      }
+      __syncthreads();
+    }
+    if (wave != 0) return;
+  }
+  // the maxima leave in natural units
+#pragma unroll
+  for (int a = 0; a < MAPS; ++a) m[a] *= 0.6931471805599453f;
   if (MAPS == 2 && splits == 1) {
     const float f0 = 1.0f / lsum[0], f1 = df.lam[0] / lsum[MAPS - 1];  // a row that is not valid holds no sum and is not written
     float ss = 0.f;
@@ -1107,15 +1193,15 @@ int msgl_mix_selective_scan(void* out, const void* x, int64_t ld_x, const void* 
 // both forms of the attention: MAPS = 1 with an optional sink, MAPS = 2 the difference of two maps
 namespace {
 
-template <int KC, int VC, int MAPS>
+template <int KC, int VC, int MAPS, bool SPREAD>
 int sink_mfma_launch(dim3 grid, hipStream_t s, bf16_t* out, int64_t ld_out, float* part_o, float* part_ml, const float* q, const bf16_t* k_cache,
                      const bf16_t* v_cache, const int* table, int64_t table_stride, const int* req_rows, const int* seq_lens, const int* cu_q,
                      int batch, int total_q, int H, int G, int d, int dv, float scale, int window, int keep, const float* sink, DiffOut df,
                      int QT, int HB, int splits) {
   const size_t lds = (size_t)kNKT * ((MAPS * KC * 32 + 8) + (VC * 16 + 8)) * sizeof(uint16_t);
   const int kvec = (((uintptr_t)k_cache & 15u) == 0 && d % 8 == 0) ? 1 : 0, vvec = (((uintptr_t)v_cache & 15u) == 0 && dv % 8 == 0) ? 1 : 0;
-  MIX_REQUIRE(ensure_lds((const void*)sink_attn_mfma_kernel<KC, VC, MAPS>, lds) == 0, "sink_attn: LDS request refused");
-  hipLaunchKernelGGL((sink_attn_mfma_kernel<KC, VC, MAPS>), grid, dim3(256), lds, s, out, ld_out, part_o, part_ml, q, k_cache, v_cache, table,
+  MIX_REQUIRE(ensure_lds((const void*)sink_attn_mfma_kernel<KC, VC, MAPS, SPREAD>, lds) == 0, "sink_attn: LDS request refused");
+  hipLaunchKernelGGL((sink_attn_mfma_kernel<KC, VC, MAPS, SPREAD>), grid, dim3(256), lds, s, out, ld_out, part_o, part_ml, q, k_cache, v_cache, table,
                      table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d, dv, scale, window, keep, sink, df, QT, HB, splits, kvec,
                      vvec);
   MIX_LAUNCHED("sink_attn (matrix cores)");
@@ -1152,15 +1238,18 @@ int sink_attn_any(void* out, int64_t ld_out, const float* q, const void* k_cache
     // matrix-core kernel: the smallest (KC, VC) instance that holds d <= 32 KC and dv <= 16 VC
     int HBm = 1;
     while (HBm * 2 <= rep && HBm * 2 <= 64) HBm *= 2;
-    const int QTm = 64 / HBm, hbl = (rep + HBm - 1) / HBm;
+    // few rows per request (decode): 16 rows per workgroup, the tiles' keys spread over its waves
+    const bool spread = HBm <= 16 && total_q <= batch * (16 / HBm);
+    const int QTm = (spread ? 16 : 64) / HBm, hbl = (rep + HBm - 1) / HBm;
     const int groups_m = (total_q + QTm - 1) / QTm + batch;
     MIX_REQUIRE((int64_t)G * hbl <= 65535, "sink_attn: too many heads");
     const dim3 grid(groups_m, G * hbl, splits);
 #define SINK_CASE(KC, VC)                                                                                                                  \
   if (d <= KC * 32 && dv <= VC * 16) {                                                                                                     \
-    const int rc = sink_mfma_launch<KC, VC, MAPS>(grid, s, mp<bf16_t>(out), ld_out, part_o, part_ml, q, cp<bf16_t>(k_cache),               \
-                                                  cp<bf16_t>(v_cache), table, table_stride, req_rows, seq_lens, cu_q, batch, total_q, H,   \
-                                                  G, d, dv, scale, window, keep, sink, df, QTm, HBm, splits);                              \
+    const auto launch = spread ? sink_mfma_launch<KC, VC, MAPS, true> : sink_mfma_launch<KC, VC, MAPS, false>;                             \
+    const int rc = launch(grid, s, mp<bf16_t>(out), ld_out, part_o, part_ml, q, cp<bf16_t>(k_cache), cp<bf16_t>(v_cache), table,           \
+                          table_stride, req_rows, seq_lens, cu_q, batch, total_q, H, G, d, dv, scale, window, keep, sink, df, QTm, HBm,    \
+                          splits);                                                                                                         \
     return rc ? rc : sink_merge_launch<bf16_t, MAPS>(s, mp<bf16_t>(out), ld_out, part_o, part_ml, total_q, H, dv, splits, sink, df);       \
   }
     if constexpr (MAPS == 1) {

@@ -416,7 +416,7 @@ __global__ __launch_bounds__(256) void postnorm_kernel(const float* __restrict__
   if (!ROUTE) return;
   float* sc = red + 4;
   __syncthreads();
-  router_logits256(srow, router, E, W, sc);
+  router_logits<4>(srow, router, E, W, sc);
   __syncthreads();
   if (threadIdx.x < 64)
     select_experts_wave<T>(sc, sc + E, sc + 2 * E, bias, E, top, G, keep, RouteRule{0, 1, 1.0f}, ids + (size_t)t * top, wts + (size_t)t * top);
@@ -426,50 +426,60 @@ __global__ __launch_bounds__(256) void postnorm_kernel(const float* __restrict__
 // seg[e] .. seg[e + 1] = the sorted positions of expert e; perm[position] = flat (token * top + choice), in flat order inside a
 // segment (stable: the layout does not depend on scheduling).  Two launches of one workgroup per expert, no atomics and nothing
 // to clear: first every expert counts its entries, then it adds up the counts before it and places its entries by a running
-// workgroup-wide rank.
-__device__ __forceinline__ int block_rank256(bool flag, int* wsum, int& total) {
-  const unsigned long long bal = __ballot(flag);
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int before = __popcll(bal & ((1ull << lane) - 1ull));
-  __syncthreads();
-  if (lane == 0) wsum[wave] = __popcll(bal);
-  __syncthreads();
-  int off = 0;
-  for (int w = 0; w < wave; ++w) off += wsum[w];
-  total = wsum[0] + wsum[1] + wsum[2] + wsum[3];
-  return off + before;
+// workgroup-wide rank (a thread looks at kSortPer consecutive entries per round).
+constexpr int kSortPer = 8;  // consecutive entries per thread and round
+
+// entries i0 + tid * kSortPer .. that belong to expert e, as a bit mask
+__device__ __forceinline__ uint32_t sort_mask(const int* __restrict__ ids, int i0, int n, int e) {
+  uint32_t m = 0;
+  const int i = i0 + threadIdx.x * kSortPer;
+#pragma unroll
+  for (int u = 0; u < kSortPer; ++u) m |= (uint32_t)(i + u < n && ids[i + u] == e) << u;
+  return m;
 }
 
 __global__ __launch_bounds__(256) void moe_count_kernel(int* __restrict__ counts, const int* __restrict__ ids, int n) {
   __shared__ int wsum[4];
   const int e = blockIdx.x;
   int cnt = 0;
-  for (int i0 = 0; i0 < n; i0 += 256) {
-    const int i = i0 + threadIdx.x;
-    int tot;
-    block_rank256(i < n && ids[i] == e, wsum, tot);
-    cnt += tot;
-  }
-  if (threadIdx.x == 0) counts[e] = cnt;
+  for (int i0 = 0; i0 < n; i0 += 256 * kSortPer) cnt += __popc(sort_mask(ids, i0, n, e));
+#pragma unroll
+  for (int o = 32; o >= 1; o >>= 1) cnt += __shfl_xor(cnt, o, 64);
+  if ((threadIdx.x & 63) == 0) wsum[threadIdx.x >> 6] = cnt;
+  __syncthreads();
+  if (threadIdx.x == 0) counts[e] = wsum[0] + wsum[1] + wsum[2] + wsum[3];
 }
 
 __global__ __launch_bounds__(256) void moe_place_kernel(int* __restrict__ seg, int* __restrict__ perm, const int* __restrict__ counts,
                                                         const int* __restrict__ ids, int n, int E) {
   __shared__ int wsum[4];
-  const int e = blockIdx.x;
+  const int e = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   int base = 0;
-  for (int k = 0; k < e; ++k) base += counts[k];
+  for (int k = lane; k < e; k += 64) base += counts[k];
+#pragma unroll
+  for (int o = 32; o >= 1; o >>= 1) base += __shfl_xor(base, o, 64);
   if (threadIdx.x == 0) {
     seg[e] = base;
     if (e == E - 1) seg[E] = base + counts[e];
   }
-  for (int i0 = 0; i0 < n; i0 += 256) {
-    const int i = i0 + threadIdx.x;
-    const bool mine = i < n && ids[i] == e;
-    int tot;
-    const int rank = block_rank256(mine, wsum, tot);
-    if (mine) perm[base + rank] = i;
-    base += tot;
+  for (int i0 = 0; i0 < n; i0 += 256 * kSortPer) {
+    const uint32_t mask = sort_mask(ids, i0, n, e);
+    const int mine = __popc(mask);
+    int upto = mine;  // inclusive prefix over the wave's lanes
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int v = __shfl_up(upto, o, 64);
+      if (lane >= o) upto += v;
+    }
+    __syncthreads();
+    if (lane == 63) wsum[wave] = upto;
+    __syncthreads();
+    int at = base + upto - mine;
+    for (int w = 0; w < wave; ++w) at += wsum[w];
+#pragma unroll
+    for (int u = 0; u < kSortPer; ++u)
+      if (mask >> u & 1u) perm[at++] = i0 + threadIdx.x * kSortPer + u;
+    base += wsum[0] + wsum[1] + wsum[2] + wsum[3];
   }
 }
 

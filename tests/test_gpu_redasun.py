@@ -507,28 +507,32 @@ def test_greedy_generation_through_the_scheduler(graphs):
     assert compared >= 2 * n_new
 
 
-def test_decode_graph_replays_bf16():
-    """A captured decode step replayed several times, eager work and synchronizations between, equals the eager step bit for bit."""
-    eng, state = engine_for(FULL, torch.bfloat16, graphs=[2], seed=12)
-    toks = {r: tokens_of(20 + 7 * i, FULL["vocab"], 80 + i) for i, r in enumerate("ab")}
-    from mini_sglang_amd.offline import OfflineRunner
-    from mini_sglang_amd.core import SamplingParams
+WIDE = config([att(heads=8, kv_heads=2, dim=64, vdim=128, dims=64, mlp=dense(ff=2048)),
+               att(heads=4, kv_heads=4, dim=32, vdim=64, dims=32, mlp=moe(experts=16, top=4, count=4, keep=2, ff=256, shared=512))],
+              width=1024, vocab=1500, loop=(0, 2, 2), embed=30.0)
 
-    sp = [SamplingParams(temperature=0.0, max_tokens=8, ignore_eos=True)] * 2
+
+@pytest.mark.parametrize("cfg", [FULL, WIDE], ids=["small", "wide"])
+def test_decode_graph_replays_bf16(cfg):
+    """Captured decode steps replayed several times, eager steps and synchronizations between, draw the tokens the eager steps draw."""
+    from mini_sglang_amd.core import SamplingParams
+    from mini_sglang_amd.offline import OfflineRunner
+
+    eng, _ = engine_for(cfg, torch.bfloat16, graphs=[2], seed=12, spaced=True)
+    prompts = [tokens_of(20, cfg["vocab"], 80), tokens_of(27, cfg["vocab"], 81)]
+    gr = eng.graph_runner
+    captured = gr.can_use_cuda_graph
     outs = []
-    for use in (True, False, True):
-        gr = eng.graph_runner
-        keep = gr.can_use_cuda_graph
-        if not use:
-            gr.can_use_cuda_graph = lambda batch: False
-        try:
+    try:
+        for use in (True, False, True, True, False):
+            gr.can_use_cuda_graph = captured if use else (lambda batch: False)
             run = OfflineRunner(eng, max_extend_tokens=64, seed=2)
-            run.generate([toks["a"], toks["b"]], sp)
+            run.generate(prompts, [SamplingParams(temperature=0.0, max_tokens=16, ignore_eos=True)] * 2)
             outs.append([run.output_ids(st) for st in run.last_states])
-        finally:
-            gr.can_use_cuda_graph = keep
-        torch.cuda.synchronize()
-    assert outs[0] == outs[1] == outs[2]
+            torch.cuda.synchronize()
+    finally:
+        gr.can_use_cuda_graph = captured
+    assert all(o == outs[0] for o in outs[1:])
 
 
 def test_generate_command(tmp_path, capsys):

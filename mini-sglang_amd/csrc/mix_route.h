@@ -19,10 +19,10 @@ struct RouteRule {
   float scale;
 };
 
-__device__ __forceinline__ float group_score(const float* c, int st, int per, int group_best) {
+__device__ __forceinline__ float group_score(const float* c, int per, int group_best) {
   float a = -INFINITY, b = -INFINITY;  // the largest and the second largest
   for (int e = 0; e < per; ++e) {
-    const float v = c[e * st];
+    const float v = c[e];
     if (v > a) {
       b = a;
       a = v;
@@ -33,71 +33,14 @@ __device__ __forceinline__ float group_score(const float* c, int st, int per, in
   return group_best == 2 && per > 1 ? a + b : a;
 }
 
-// One thread, one token: s[e * st] holds the logits on entry (st = column stride), c is scratch of the same shape, gs of G entries.
-template <typename T>
-__device__ __forceinline__ void select_experts(float* s, float* c, float* gs, int st, const T* __restrict__ bias, int E, int top, int G,
-                                               int keep, RouteRule rule, int* __restrict__ ids, float* __restrict__ wts) {
-  if (rule.sigmoid) {
-    for (int e = 0; e < E; ++e) {
-      const float v = 1.0f / (1.0f + expf(-s[e * st]));
-      s[e * st] = v;
-      c[e * st] = v + (bias ? ld(bias + e) : 0.f);
-    }
-  } else {
-    float mx = -INFINITY;
-    for (int e = 0; e < E; ++e) mx = fmaxf(mx, s[e * st]);
-    float sum = 0.f;
-    for (int e = 0; e < E; ++e) {
-      const float v = expf(s[e * st] - mx);
-      s[e * st] = v;
-      sum += v;
-    }
-    for (int e = 0; e < E; ++e) {
-      const float v = s[e * st] / sum;
-      s[e * st] = v;
-      c[e * st] = v + (bias ? ld(bias + e) : 0.f);
-    }
-  }
-  const int per = E / G;
-  if (keep < G) {
-    // a group stays if fewer than `keep` groups beat it (ties: the lower index wins)
-    for (int g = 0; g < G; ++g) gs[g * st] = group_score(c + g * per * st, st, per, rule.group_best);
-    for (int g = 0; g < G; ++g) {
-      const float mine = gs[g * st];
-      int better = 0;
-      for (int o2 = 0; o2 < G; ++o2) better += (gs[o2 * st] > mine) || (gs[o2 * st] == mine && o2 < g);
-      if (better >= keep)
-        for (int e = g * per; e < (g + 1) * per; ++e) c[e * st] = -INFINITY;
-    }
-  }
-  float tot = 0.f;
-  for (int k = 0; k < top; ++k) {
-    int best = -1;
-    float bv = -INFINITY;
-    for (int e = 0; e < E; ++e) {
-      const float v = c[e * st];
-      if (v > bv) {
-        best = e;
-        bv = v;
-      }
-    }
-    if (best < 0) best = 0;  // unreachable: the host checks top <= keep * (E / G) and choice scores are finite
-    ids[k] = best;
-    const float sv = s[best * st];
-    wts[k] = sv;
-    tot += sv;
-    c[best * st] = -INFINITY;
-  }
-  for (int k = 0; k < top; ++k) wts[k] = wts[k] / (tot + 1e-20f) * rule.scale;
-}
-
 __device__ __forceinline__ float wave_max_f(float v) {
 #pragma unroll
   for (int o = 32; o >= 1; o >>= 1) v = fmaxf(v, __shfl_xor(v, o, 64));
   return v;
 }
 
-// The same by the 64 lanes of one wave over one token (lane owns experts lane, lane + 64, ...).  s, c: E entries of LDS each, gs: G + top.
+// The 64 lanes of one wave over one token (lane owns experts lane, lane + 64, ...).  s: the E logits on entry; s, c: E entries of LDS each,
+// gs: G + top.
 template <typename T>
 __device__ __forceinline__ void select_experts_wave(float* s, float* c, float* gs, const T* __restrict__ bias, int E, int top, int G,
                                                     int keep, RouteRule rule, int* __restrict__ ids, float* __restrict__ wts) {
@@ -127,7 +70,7 @@ __device__ __forceinline__ void select_experts_wave(float* s, float* c, float* g
   }
   const int per = E / G;
   if (keep < G) {
-    for (int g = lane; g < G; g += 64) gs[g] = group_score(c + g * per, 1, per, rule.group_best);
+    for (int g = lane; g < G; g += 64) gs[g] = group_score(c + g * per, per, rule.group_best);
     for (int g = lane; g < G; g += 64) {
       const float mine = gs[g];
       int better = 0;

@@ -15,7 +15,7 @@
 //   lightning_kernel         S <- decay * S + k v^T, o = S^T q per (request, head), state rows indexed by slot; long portions
 //                            as parallel chunks joined by lightning_scan_kernel
 //   gated_norm_kernel        rms over the concatenated heads * w * sigmoid(g)
-//   route_kernel             fp32 router on fp32 logits: softmax, bias-corrected group-limited top-k, normalised weights
+//   route_kernel             fp32 router on fp32 logits (mix_route.h): softmax or sigmoid, bias-corrected group-limited top-k, normalised weights
 //   moe_count / moe_place    (token, choice) pairs bucketed by expert -> segment offsets + permutation
 //   gemm_nt_mfma_kernel      grouped / segmented / gathered C = act(A B^T) for 16-bit weights on the matrix cores: per-head
 //                            latent products, expert layers, router logits of long batches
@@ -364,22 +364,17 @@ __global__ __launch_bounds__(256) void gated_norm_kernel(T* __restrict__ out, co
 }
 
 // ------------------------------------------------------------------------------------------------ router
-// One thread per token over router logits z [T, E] that a product kernel wrote in fp32 (bf16 x bf16 products are exact in fp32,
-// so the matrix cores' fp32 accumulation IS the 32-bit router on the token's 16-bit copy); scores, choice and weights as in mix_route.h.
-// Scores live in LDS columns, one per thread.
+// One wave per token over router logits z [T, E] that a product wrote in fp32 (bf16 x bf16 products are exact in fp32, so the matrix
+// cores' fp32 accumulation IS the 32-bit router on the token's 16-bit copy); scores, choice and weights as in mix_route.h.
 template <typename T>
-__global__ __launch_bounds__(64) void route_kernel(int* __restrict__ ids, float* __restrict__ wts, const float* __restrict__ z,
-                                                   const T* __restrict__ bias, int tokens, int E, int top, int G, int keep, RouteRule rule,
-                                                   int TPB) {
+__global__ __launch_bounds__(256) void route_kernel(int* __restrict__ ids, float* __restrict__ wts, const float* __restrict__ z,
+                                                    const T* __restrict__ bias, int tokens, int E, int top, int G, int keep, RouteRule rule) {
   extern __shared__ float lds[];
-  const int t = blockIdx.x * TPB + threadIdx.x;
-  if (threadIdx.x >= TPB || t >= tokens) return;
-  float* s = lds + threadIdx.x;             // s[e * TPB]
-  float* c = lds + (size_t)E * TPB + threadIdx.x;
-  const float* zr = z + (size_t)t * E;
-#pragma unroll 8
-  for (int e = 0; e < E; ++e) s[e * TPB] = zr[e];
-  select_experts<T>(s, c, c + (size_t)E * TPB, TPB, bias, E, top, G, keep, rule, ids + (size_t)t * top, wts + (size_t)t * top);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, t = blockIdx.x * (blockDim.x >> 6) + wave;
+  if (t >= tokens) return;  // whole waves; no barrier below
+  float* s = lds + (size_t)wave * (2 * E + G + top);
+  for (int e = lane; e < E; e += 64) s[e] = z[(size_t)t * E + e];
+  select_experts_wave<T>(s, s + E, s + 2 * E, bias, E, top, G, keep, rule, ids + (size_t)t * top, wts + (size_t)t * top);
 }
 
 template <typename T, bool ROUTE>
@@ -1092,13 +1087,13 @@ int msgl_mix_route(int* ids, float* wts, const float* z, const void* bias, int t
               "route: bad sizes E %d top %d groups %d keep %d", E, top, G, keep);
   MIX_REQUIRE(group_best == 1 || group_best == 2, "route: a group's score sums its 1 or 2 largest choices, not %d", group_best);
   if (tokens == 0) return MSGL_MIX_OK;
-  int tpb = 64;
-  while (tpb > 1 && (size_t)(2 * E + G) * tpb * sizeof(float) > 64 * 1024) tpb >>= 1;
-  const size_t lds = (size_t)(2 * E + G) * tpb * sizeof(float);
+  int waves = 4;
+  while (waves > 1 && (size_t)(2 * E + G + top) * waves * sizeof(float) > 64 * 1024) waves >>= 1;
+  const size_t lds = (size_t)(2 * E + G + top) * waves * sizeof(float);
   MIX_REQUIRE(lds <= 64 * 1024, "route: too many experts");
   hipStream_t s = static_cast<hipStream_t>(stream);
-  DISPATCH_T(dtype, hipLaunchKernelGGL(route_kernel<T>, dim3((tokens + tpb - 1) / tpb), dim3(64), lds, s, ids, wts, z, cp<T>(bias), tokens, E,
-                                       top, G, keep, RouteRule{sigmoid, group_best, scale}, tpb);)
+  DISPATCH_T(dtype, hipLaunchKernelGGL(route_kernel<T>, dim3((tokens + waves - 1) / waves), dim3(64 * waves), lds, s, ids, wts, z, cp<T>(bias),
+                                       tokens, E, top, G, keep, RouteRule{sigmoid, group_best, scale});)
   MIX_LAUNCHED("route");
   return MSGL_MIX_OK;
 }

@@ -181,7 +181,7 @@ def route(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], t
     assert h.is_contiguous() and router.is_contiguous() and router.shape == (E, W) and router.dtype == h.dtype
     assert bias is None or (bias.dtype == h.dtype and bias.shape == (E,) and bias.is_contiguous())
     z = torch.empty((T, E), dtype=torch.float32, device=h.device)
-    gemm_nt(z, h, router, T, E, W, lda=W, ldb=W, ldc=E)
+    linear(h, router, out=z)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=h.device)
     check_mix(mix_lib().msgl_mix_route(ids.data_ptr(), wts.data_ptr(), z.data_ptr(), _p(bias), T, E, top, groups, keep, int(sigmoid),
@@ -333,7 +333,7 @@ def route_top(h: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
     assert h.is_contiguous() and router.is_contiguous() and router.shape == (E, W) and router.dtype == h.dtype
     assert bias is None or (bias.dtype == h.dtype and bias.shape == (E,) and bias.is_contiguous())
     z = torch.empty((T, E), dtype=torch.float32, device=h.device)
-    gemm_nt(z, h, router, T, E, W, lda=W, ldb=W, ldc=E)
+    linear(h, router, out=z)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=h.device)
     check_mix(mix_lib().msgl_mix_route_top(ids.data_ptr(), wts.data_ptr(), z.data_ptr(), _p(bias), T, E, top, _code(h), _stream()),
@@ -754,7 +754,7 @@ def route_sigmoid(h: torch.Tensor, router: torch.Tensor, top: int):
     E = router.shape[0]
     assert h.is_contiguous() and router.is_contiguous() and router.shape == (E, W) and router.dtype == h.dtype
     z = torch.empty((T, E), dtype=torch.float32, device=h.device)
-    gemm_nt(z, h, router, T, E, W, lda=W, ldb=W, ldc=E)
+    linear(h, router, out=z)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
     wts = torch.empty((T, top), dtype=torch.float32, device=h.device)
     check_mix(mix_lib().msgl_mix_route_sigmoid(ids.data_ptr(), wts.data_ptr(), z.data_ptr(), T, E, top, _stream()), "route_sigmoid")

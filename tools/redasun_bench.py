@@ -112,7 +112,7 @@ def kernel_rooflines(name: str, prompt: int, batch: int, device) -> dict:
         win = rnd(W, 2 * W, scale=W ** -0.5)
         put("loop product (fp32 result)", lambda: mixops.linear(wide, win, out=x2), 4.0 * T * W * W, W * W * 4 + T * W * (4 + 4))
         put("loop product (16-bit result, like)", lambda: mixops.linear(wide, win, out=h), 4.0 * T * W * W, W * W * 4 + T * W * (4 + 2))
-        # --- router (like: largest logits, sigmoid weights, expert inputs scaled in the same launch / by a launch of its own)
+        # --- router (like: largest logits, sigmoid weights; in short steps expert inputs scaled in the same launch)
         router, corr = rnd(E, W, scale=W ** -0.5), rnd(E, scale=0.1)
         rule = (top, groups, keep, True, 2, 2.0)
         if T <= 128:
@@ -128,11 +128,7 @@ def kernel_rooflines(name: str, prompt: int, batch: int, device) -> dict:
             byts = T * W * 2 + E * W * 2 + T * E * 8
             put("route", lambda: mixops.route(h, router, corr, top, groups, keep, sigmoid=True, group_best=2, scale=2.0), 2.0 * T * W * E, byts)
 
-            def like():
-                _, wt = mixops.route_sigmoid(h, router, top)
-                mixops.scale_rows(h, wt)
-
-            put("route_sigmoid, scale_rows (like)", like, 2.0 * T * W * E, byts + T * W * 2 * (1 + top))
+            put("route_sigmoid (like)", lambda: mixops.route_sigmoid(h, router, top), 2.0 * T * W * E, byts)
         # --- gated activation (like: the clamped gate)
         gu = rnd(T, 2 * ff)
         put("gate_mul (gelu)", lambda: mixops.gate_mul(gu, mixops.GATE_MUL_GELU_TANH), 0.0, T * ff * 6)

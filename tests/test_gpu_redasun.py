@@ -377,7 +377,7 @@ def test_one_loud_key_far_back(dev, dtype, loud, loud_map):
 
 
 @pytest.mark.parametrize("H,G,d,dv", [(4, 4, 32, 64), (8, 2, 64, 64), (6, 3, 40, 40), (3, 1, 64, 128), (16, 2, 128, 128), (2, 1, 100, 104), (8, 1, 128, 256),
-                                      (5, 5, 72, 136), (2, 1, 160, 96), (4, 2, 7, 9), (2, 1, 20, 300), (5, 1, 44, 92), (7, 1, 24, 48), (1, 1, 130, 520)])
+                                      (5, 5, 72, 136), (2, 1, 160, 96), (4, 2, 7, 9), (2, 1, 20, 300), (5, 1, 44, 92), (7, 1, 24, 48), (1, 1, 130, 520), (34, 1, 16, 32), (40, 2, 64, 112)])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16], ids=["fp32", "bf16"])
 def test_two_map_attention_head_sizes(dev, dtype, H, G, d, dv):
     """Every matrix-core instance (and the plain kernel beside it): a portion, single tokens, a portion of two, the rest; keys in one range and in three."""
